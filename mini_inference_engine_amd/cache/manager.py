@@ -10,7 +10,8 @@ ceil((computed + n) / page) - len(table); reservation is all-or-nothing with an
 optional watermark; everything a request holds goes back when it ends or is
 preempted.  Beyond the reference: a windowed group also gives back pages that
 lie wholly before the window once a step has passed them (their table entries
-become 0, the scratch page), and every request holds a state slot.
+become 0, the scratch page), except those of a request's first tokens that the
+group keeps, and every request holds a state slot.
 """
 from __future__ import annotations
 
@@ -33,6 +34,7 @@ class RequestCache:
 class GroupSpec:
     window: int | None
     num_pages: int
+    keep_first: int = 0              # beside a window: first tokens of a request that every later query sees
 
 
 class CacheManager:
@@ -119,8 +121,9 @@ class CacheManager:
                 continue
             # the next query sits at position >= num_computed and sees keys >= num_computed - w + 1
             first = min(max(0, num_computed - spec.window + 1) // self.page_size, len(rc.tables[g]))
+            kept = -(-spec.keep_first // self.page_size)        # pages that hold a kept first token
             gone = []
-            for i in range(rc.first_live[g], first):
+            for i in range(max(rc.first_live[g], kept), first):
                 if rc.tables[g][i] != 0:
                     gone.append(rc.tables[g][i])
                     rc.tables[g][i] = 0

@@ -60,6 +60,8 @@ class StepContext:
     max_row_tokens: int = 0          # longest row (host)
     max_context: int = 0             # largest row_context (host), or a static bound when captured
     host: dict = field(default_factory=dict)   # the same arrays as numpy, for parts that plan on the host
+    shared: dict = field(default_factory=dict)  # what one layer of the step leaves for later ones, by name (tensors over the
+                                                # step's tokens; a layer that gives writes it anew in every forward)
 
 
 class StepArena:

@@ -91,7 +91,8 @@ class ModelRunner:
             num_pages = max(2, budget // max(1, sum(per_page))) if n_groups else 2
         self.num_pages = int(num_pages)
         self.num_state_slots = int(num_state_slots or max_rows + 1)
-        self.cache = CacheManager(page_size, [GroupSpec(w, self.num_pages) for w in self.model.page_groups],
+        self.cache = CacheManager(page_size, [GroupSpec(w, self.num_pages, k) for w, k in zip(self.model.page_groups,
+                                                                                            self.model.page_group_keeps)],
                                   self.num_state_slots)
         self.storage = CacheStorage(self.model, page_size, [self.num_pages] * n_groups, self.num_state_slots,
                                     self.device, self.dtype)

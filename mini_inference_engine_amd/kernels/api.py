@@ -140,6 +140,11 @@ class KernelBackend:
             return self.linear_silu_mul(x, w_gate_up, intermediate)
         raise NotImplementedError
 
+    def linear_clamped_glu(self, x, w_gate_up, intermediate, limit, alpha, shift):
+        """gu = x w^T with w [2 * intermediate, in]; returns g * sigmoid(alpha g) * (u + shift) with g = min(gu[:, :I], limit),
+        u = clamp(gu[:, I:], -limit, limit) -> [T, I] in the activation dtype.  ``x`` is a tensor or a Normed."""
+        raise NotImplementedError
+
     def linear_act(self, x, w, activation="relu2"):
         """act(x w^T), act one of ACTIVATIONS, computed on the product's 32-bit sums and rounded once
         -> [T, out] in the activation dtype.  ``x`` is a tensor or a Normed."""
@@ -276,7 +281,8 @@ class KernelBackend:
 
     def qkv_finish(self, sums, q_col, k_col, v_col, num_q_heads, num_kv_heads, dim, vdim, padded_dim, positions, inv_freq,
                    layout, k_cache, v_cache, slot_mapping, q_norm=None, k_norm=None, eps=0.0, q_head_scale=None,
-                   norm_per_head=False, col_bias=None, position_temperature=None):
+                   norm_per_head=False, col_bias=None, position_temperature=None, rotation_scale=1.0, conv=None,
+                   values_out=None, value_mix=None):
         """What lies between a q/k/v projection's float32 sums [T, *] and attention, in 32-bit: queries are columns
         [q_col, q_col + Hq dim), keys [k_col, k_col + Hkv dim), values [v_col, v_col + Hkv vdim), or, with ``v_col``
         None, the keys as projected (vdim = dim).  ``col_bias`` (float32, one number a column of the sums): the
@@ -289,12 +295,51 @@ class KernelBackend:
         "interleaved" pairs (2i, 2i + 1), "half" pairs (i, i + len(inv_freq)).  ``q_head_scale`` (float32 [Hq]):
         head h's turned query times that number.  Keys and values go to the token's slot of k_cache [pages, Hkv, page, P]
         and v_cache [pages, Hkv, P, page], P = ``padded_dim`` >= dim, vdim, zeros beyond their own size.
+        ``conv`` = (taps, tail, step): before anything else every channel c of the three projections, which then lie side by
+        side from q_col on (C = (Hq + Hkv) dim + Hkv vdim of them), passes y_t = sum_j taps[c, j] u_(t - K + 1 + j) (taps float32
+        [C, K]) over its row's tokens; inputs before the row's first token come from ``tail`` [slots, max(1, K - 1), C] float32,
+        which moves on (as in ``residual_conv``).  ``rotation_scale``: factor on every cosine and sine.  ``values_out`` (float32
+        [T, Hkv vdim]) receives the values; ``value_mix`` = (lam, other float32 [T, Hkv vdim]): what is cached as values is
+        (1 - lam) v + lam other.
         -> q [T, Hq * P] in the activation dtype, zeros beyond dim."""
         raise NotImplementedError
 
     def head_gate_(self, o, gate, gate_col, num_heads, head_dim):
         """o [T, H * head_dim] *= sigmoid(gate[t, gate_col + h]) for every number of head h, in place (gate float32
         [T, *]).  Returns o."""
+        raise NotImplementedError
+
+    def gate_heads(self, o, gate, gate_col, num_heads, vdim, padded_dim, out=None, scale=1.0):
+        """o [T, H padded_dim] -> scale * o[t, h, :vdim] * sigmoid(gate[t, gate_col + h vdim + ...]) [T, H vdim], into ``out``
+        (rows may be further apart than H vdim) or a new tensor; gate float32 [T, *]."""
+        raise NotImplementedError
+
+    # ---- recurrences with one decay a head and token
+    def short_conv(self, x, col, channels, taps, bias, tail, step, activation="none"):
+        """u[t, c] = act(bias[c] + sum_j taps[c, j] x[t - (K - 1) + j, col + c]) over each row's tokens (x float32 [T, *], taps
+        float32 [C, K], bias float32 [C] or None; act "none" or one of ACTIVATIONS); inputs before a row's first token come
+        from ``tail`` [slots, max(1, K - 1), C] float32, which moves on (as in ``residual_conv``).  -> [T, C] float32."""
+        raise NotImplementedError
+
+    def state_space(self, u, b_col, c_col, sums, z_col, dt_col, num_heads, groups, state_dim, vdim, dt_bias, rate, skip,
+                    norm_groups, norm_weight, eps, state, step, out=None, scale=1.0):
+        """Mamba-2's recurrence and gated norm.  u [T, *] float32: x in columns [0, H vdim), B from b_col, C from c_col on
+        (groups * state_dim each; head h reads group h // (H / groups)); sums float32 [T, *]: the gate z from z_col (H vdim), dt from
+        dt_col (H).  dt <- softplus(dt + dt_bias); per row and head, tokens in order, from the row's slot of ``state`` [slots,
+        H, state_dim, vdim] float32, left there afterwards: S <- exp(-rate dt) S + dt B x^T; y = S^T C + skip x.  Then y silu(z),
+        RMS-normed in ``norm_groups`` equal parts of H vdim, times norm_weight, times scale -> [T, H vdim] in the activation
+        dtype, into ``out`` (rows may be further apart) or a new tensor."""
+        raise NotImplementedError
+
+    def mlstm(self, sums, cols, num_heads, dim, vdim, i_bias, f_bias, cap, q_scale, norm_weight, eps, state, normaliser, maximum,
+              step, out=None, scale=1.0):
+        """Matrix memory with exponential gates, from one product's float32 sums [T, *].  ``cols``: first column of q, k (H dim
+        each), v and the output gate g (H vdim each), i and f (H each).  i = cap tanh((i + i_bias) / cap), f = logsigmoid(cap
+        tanh((f + f_bias) / cap)); per row and head, tokens in order, from the row's slot of ``state`` [slots, H, dim, vdim],
+        ``normaliser`` [slots, H, dim] and ``maximum`` [slots, H], float32, left there afterwards: m' = max(f + m, i);
+        S <- exp(f + m - m') S + exp(i - m') k v^T, n likewise with k alone; o = S^T q / (max(|n . q|, exp(-m')) + 1e-6) with
+        q times q_scale.  -> scale * rmsnorm(o over a head, eps) * norm_weight [H vdim] * sigmoid(g) [T, H vdim] in the
+        activation dtype, into ``out`` (rows may be further apart) or a new tensor."""
         raise NotImplementedError
 
     def delta_rule(self, sums, cols, num_heads, dim, w_decay, decay_bias, decay_scale, removal_bias, norm_weight, eps,
@@ -346,12 +391,13 @@ class KernelBackend:
 
     def paged_attention(self, qkv, num_q_heads, num_kv_heads, head_dim, k_cache, v_cache, group, step, scale,
                         window, sink=None, weights="softmax", softcap=None, chunk=None, head_bias=None,
-                        distance_bias=None):
+                        distance_bias=None, keep_first=0):
         """For token t of row r at position p: softmax over keys max(0, p - window + 1)..p
         of row r (read through group.block_tables[r]) of (q . k) * scale, times v.
         q head i uses kv head i // (Hq / Hkv).  q is the first Hq * D columns of
-        qkv (row stride qkv.stride(0)).  ``sink`` (a number): one more term exp(sink) in every softmax's
-        denominator, with no value.  ``chunk`` (a number of positions): keys before floor(p / chunk) * chunk are not
+        qkv (row stride qkv.stride(0)).  ``keep_first``: beside the window keys 0 .. keep_first - 1 (up to p) are seen too.
+        ``sink`` (a number, or float32 [Hq], one a query head): one more term exp(sink) in every softmax's denominator, with
+        no value.  ``chunk`` (a number of positions): keys before floor(p / chunk) * chunk are not
         seen either.  ``softcap`` (c > 0): the scaled scores pass through c * tanh(score / c).  ``weights`` "sigmoid":
         no softmax; a visible key counts with sigmoid(score + head_bias[i]) (head_bias float32 [Hq] or None), not
         normalised over the keys (no sink).  ``distance_bias`` (float32 [Hq, N]): a key n positions back of the query

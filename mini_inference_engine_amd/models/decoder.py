@@ -27,6 +27,7 @@ class Decoder:
         # cache needs, one per owning run-order entry; groups by window
         self.cache_entries: dict[int, CacheEntry] = {}
         self.page_groups: list = []       # window (None = all keys) of each page group
+        self.page_group_keeps: list = []  # first tokens of a request each page group keeps beside its window
         group_keys: list = []
         for e, call in enumerate(spec.schedule):
             if call.cache_of is not None:
@@ -42,6 +43,7 @@ class Decoder:
                 if key not in group_keys:
                     group_keys.append(key)
                     self.page_groups.append(req.window)
+                    self.page_group_keeps.append(req.keep_first)
                 ce.group = group_keys.index(key)
             self.cache_entries[e] = ce
         self.bindings: list[CacheBinding] = []

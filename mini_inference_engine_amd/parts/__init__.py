@@ -11,12 +11,15 @@ from .gla import GatedLinearAttention
 from .input_conv import ConvTail, ResidualConv
 from .latent_attention import LatentAttention, PagedLatent
 from .layernorm import LayerNorm
+from .mlstm import MatrixLSTM, MatrixMemory
 from .rglru import RGLRU, RecurrentState
 from .rmsnorm import RMSNorm
-from .rope import NoPosition, RotaryHalfAngles, RotaryHalfSplit, RotaryInterleaved, rotary_tables
+from .rope import NoPosition, RotaryHalfAngles, RotaryHalfSplit, RotaryInterleaved, RotaryYarn, rotary_tables
 from .routed_experts import RoutedExperts
+from .scaled_pair import ScaledPair
 from .side_by_side import SideBySide
 from .sigmoid_attention import SigmoidAttention
 from .softmax_attention import SoftmaxAttention
+from .state_space import StateSpace
 from .summed_ff import SummedFF
 from .swiglu import SwiGLU

@@ -143,6 +143,7 @@ class CacheRequirement:
                  whose requirements are paged can run a prompt portion in a captured step of more tokens).
     window       for paged data: how many keys back a query looks at most (None = all); pages that lie
                  wholly before the window are given back.
+    keep_first   beside a window: how many first keys of a request every query sees too; their pages stay.
     bytes_per_page(page_size, element_size)   what one page id costs in this entry (sizes the pool)
     allocate(num_pages, page_size, num_slots, device, act_dtype) -> dict of tensors, handed to the mixer as
                  CacheBinding.k / .v / .state (keys of those names) and CacheBinding.tensors (all of them)
@@ -150,6 +151,7 @@ class CacheRequirement:
     """
     paged = False
     window = None
+    keep_first = 0
 
     @property
     def stateful(self) -> bool:
@@ -162,7 +164,7 @@ class CacheRequirement:
         return list(tensors.values()) if self.paged else []
 
     def page_group_key(self):
-        return self.window
+        return (self.window, self.keep_first) if self.keep_first else self.window
 
     def bytes_per_page(self, page_size: int, element_size: int) -> int:
         return 0
@@ -176,12 +178,13 @@ class CacheRequirement:
 
 @dataclass(frozen=True)
 class PagedKV(CacheRequirement):
-    """Keys and values of every token in pages; ``window`` keys back at most, or all.  Keys
-    [pages, kv_heads, page, head_dim]; values [pages, kv_heads, head_dim, page] (a page's values transposed:
+    """Keys and values of every token in pages; ``window`` keys back at most (and the request's ``keep_first`` first
+    ones), or all.  Keys [pages, kv_heads, page, head_dim]; values [pages, kv_heads, head_dim, page] (a page's values transposed:
     both are then what the attention kernels' matrix instructions take straight from memory)."""
     num_kv_heads: int
     head_dim: int
     window: int | None = None
+    keep_first: int = 0
     paged = True
 
     def bytes_per_page(self, page_size, element_size):
@@ -239,6 +242,10 @@ class CombinedCache(CacheRequirement):
     @property
     def window(self):
         return self._paged.window if self._paged is not None else None
+
+    @property
+    def keep_first(self):
+        return self._paged.keep_first if self._paged is not None else 0
 
     @property
     def stateful(self):

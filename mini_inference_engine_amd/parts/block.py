@@ -13,14 +13,19 @@ from .base import Block, CombinedCache, register_block
 
 @register_block("pre_norm")
 class PreNormBlock(Block):
-    def __init__(self, norm_mixer, mixer, norm_feed_forward, feed_forward):
+    """``feed_forward`` (and its norm) may be None: the layer is its mixer alone, whose output is then what the block
+    leaves to be added."""
+
+    def __init__(self, norm_mixer, mixer, norm_feed_forward=None, feed_forward=None):
+        if (feed_forward is None) != (norm_feed_forward is None):
+            raise ValueError("a feed-forward and its norm come together or not at all")
         self.norm_mixer = norm_mixer
         self.mixer = mixer
         self.norm_feed_forward = norm_feed_forward
         self.feed_forward = feed_forward
 
     def children(self):
-        return [self.norm_mixer, self.mixer, self.norm_feed_forward, self.feed_forward]
+        return [p for p in (self.norm_mixer, self.mixer, self.norm_feed_forward, self.feed_forward) if p is not None]
 
     @property
     def first_norm(self):
@@ -32,6 +37,8 @@ class PreNormBlock(Block):
         y = self.norm_mixer.lazy(h, residual)
         if not self.mixer.lazy_input:
             y = y.materialize()
+        if self.feed_forward is None:
+            return self.mixer.forward(y, step, cache, add_to=_sink(residual, next_norm)), residual
         a = self.mixer.forward(y, step, cache, add_to=_sink(residual, self.norm_feed_forward))
         y = self.norm_feed_forward.lazy(a, residual)
         if not self.feed_forward.lazy_input:

@@ -8,6 +8,8 @@ The tables stay in 32-bit whatever the activation dtype is.
 """
 from __future__ import annotations
 
+import math
+
 import torch
 
 from .base import PositionEncoding, register_position_encoding
@@ -78,6 +80,7 @@ class RotaryInterleaved(PositionEncoding):
     themselves, so there is no table and no longest position."""
 
     layout = "interleaved"
+    magnitude = 1.0         # factor on every cosine and sine
 
     def __init__(self, rotary_dim: int, theta: float, factor: float = 1.0):
         """``factor``: linear scaling, every frequency divided by it."""
@@ -90,10 +93,14 @@ class RotaryInterleaved(PositionEncoding):
             raise ValueError("theta and the scaling factor must be positive")
         self.inv_freq = None
 
+    def frequencies(self):
+        """Angle a position of each pair, float64 [rotary_dim / 2]."""
+        exponent = torch.arange(0, self.rotary_dim, 2, dtype=torch.float64) / self.rotary_dim
+        return self.theta ** -exponent / self.factor
+
     def prepare(self, device, dtype):
         if self.inv_freq is None or self.inv_freq.device != torch.device(device):
-            exponent = torch.arange(0, self.rotary_dim, 2, dtype=torch.float64) / self.rotary_dim
-            self.inv_freq = (self.theta ** -exponent / self.factor).to(torch.float32).to(device).contiguous()
+            self.inv_freq = self.frequencies().to(torch.float32).to(device).contiguous()
 
 
 @register_position_encoding("rotary_half_angles")
@@ -102,3 +109,27 @@ class RotaryHalfAngles(RotaryInterleaved):
     i + rotary_dim / 2.  Like RotaryInterleaved it keeps no table: the kernels that use it compute
     position * inv_freq[i] and its cosine and sine in 32-bit themselves."""
     layout = "half"
+
+
+@register_position_encoding("rotary_yarn")
+class RotaryYarn(RotaryHalfAngles):
+    """The halves' pairing with frequencies stretched by parts (YaRN: Peng et al., "YaRN: Efficient Context Window
+    Extension of Large Language Models").  With n(t) = rotary_dim ln(original / (2 pi t)) / (2 ln theta), the place of the
+    pair that turns t times over ``original`` positions: pairs up to floor(n(fast)) keep their frequency, pairs from
+    ceil(n(slow)) on have theirs divided by ``factor``, those between move from one to the other linearly.  Cosines
+    and sines are multiplied by 0.1 ln(factor) + 1."""
+
+    def __init__(self, rotary_dim: int, theta: float, factor: float, original: float, fast: float, slow: float):
+        super().__init__(rotary_dim, theta)
+        self.stretch, self.original, self.fast, self.slow = float(factor), float(original), float(fast), float(slow)
+        if not (self.stretch > 0 and self.original > 0 and self.fast > 0 and self.slow > 0) or self.theta == 1.0:
+            raise ValueError("factor, original, fast and slow must be positive, and theta another number than 1")
+        self.magnitude = 0.1 * math.log(self.stretch) + 1.0
+
+    def frequencies(self):
+        plain = super().frequencies()
+        place = lambda turns: self.rotary_dim * math.log(self.original / (2 * math.pi * turns)) / (2 * math.log(self.theta))   # noqa: E731
+        low = max(math.floor(place(self.fast)), 0)
+        high = min(math.ceil(place(self.slow)), self.rotary_dim - 1)
+        ramp = ((torch.arange(plain.shape[0], dtype=torch.float64) - low) / max(high - low, 0.001)).clamp(0, 1)
+        return plain / self.stretch * ramp + plain * (1 - ramp)
