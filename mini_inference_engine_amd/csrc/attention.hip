@@ -13,7 +13,8 @@
 // joins the softmax's denominator at the end and has no value.  With a cap c the scaled scores
 // pass through c * tanh(score / c).  In the sigmoid mode there is no softmax: a visible key counts
 // with sigmoid(score + the head's bias), and the weights are not normalised.  With a distance bias a key n
-// positions back adds a number of its head's table to the score.
+// positions back adds a number of its head's table to the score.  With a window and kept first keys a query also
+// sees keys 0 .. keep - 1, taken before the window's.  The sink may be a number a query head.
 //
 // This is the reference kernel of the engine: the float32 path runs on it, and the
 // bfloat16 path uses it wherever a faster kernel does not take the shape.
@@ -47,7 +48,7 @@ paged_attention_kernel(const T* __restrict__ q, long q_stride, const T* __restri
                        int max_blocks, const int* __restrict__ token_row, const int* __restrict__ positions, int Hq,
                        int Hkv, int D, int page, float scale, int window, int has_sink, float sink, int chunk,
                        float softcap, int sigmoid, const float* __restrict__ head_bias,
-                       const float* __restrict__ dist_bias, int dist_n) {
+                       const float* __restrict__ dist_bias, int dist_n, int keep, const float* __restrict__ head_sinks) {
   __shared__ float qs[NR * 64];
   __shared__ float ps[64];
   __shared__ long long base[64];     // per key of the chunk: offset of its value column
@@ -69,9 +70,13 @@ paged_attention_kernel(const T* __restrict__ q, long q_stride, const T* __restri
 #pragma unroll
   for (int i = 0; i < NR; ++i) acc[i] = 0.f;
 
-  for (int c0 = lo; c0 <= pos; c0 += 64) {
+  const int kept = keep < lo ? keep : lo;             // keys [0, kept) first, then [lo, pos]
+  for (int c0 = kept > 0 ? 0 : lo, next; c0 <= pos; c0 = next) {
+    const int limit = c0 < kept ? kept : pos + 1;     // end of this stretch of keys
+    next = c0 + 64;
+    if (c0 < kept && next >= kept) next = lo;
     const int key = c0 + lane;
-    const bool valid = key <= pos;
+    const bool valid = key < limit;
     float s = -INFINITY;
     if (valid) {
       const int pg = bt[key / page];
@@ -93,7 +98,7 @@ paged_attention_kernel(const T* __restrict__ q, long q_stride, const T* __restri
     if (sigmoid) {
       p = valid ? mie_sigmoid(s + hb) : 0.f;
     } else {
-      const float m_new = fmaxf(m, wave_max(s));    // finite: key c0 <= pos is valid
+      const float m_new = fmaxf(m, wave_max(s));    // finite: key c0 < limit is valid
       alpha = expf(m - m_new);                      // 0 on the first chunk (m = -inf)
       p = valid ? expf(s - m_new) : 0.f;
       l = l * alpha + wave_sum(p);
@@ -101,7 +106,7 @@ paged_attention_kernel(const T* __restrict__ q, long q_stride, const T* __restri
     }
     ps[lane] = p;
     __syncthreads();
-    const int nk = pos - c0 + 1 < 64 ? pos - c0 + 1 : 64;
+    const int nk = limit - c0 < 64 ? limit - c0 : 64;
 #pragma unroll
     for (int i = 0; i < NR; ++i) acc[i] *= alpha;
     for (int j = 0; j < nk; ++j) {
@@ -115,6 +120,7 @@ paged_attention_kernel(const T* __restrict__ q, long q_stride, const T* __restri
     }
     __syncthreads();
   }
+  if (head_sinks) sink = head_sinks[h];
   if (has_sink && !sigmoid) {                     // one more term exp(sink) in the denominator, with no value
     const float m_new = fmaxf(m, sink);
     const float alpha = expf(m - m_new);
@@ -137,8 +143,10 @@ static int paged_attention_launch(const void* q, long q_stride, const void* k_ca
                                    int dtype, const int* block_tables, int max_blocks, const int* token_row,
                                    const int* positions, int tokens, int Hq, int Hkv, int D, int page, float scale,
                                    int window, int has_sink, float sink, int chunk, float softcap, int sigmoid,
-                                   const float* head_bias, const float* dist_bias, int dist_n, hipStream_t stream) {
+                                   const float* head_bias, const float* dist_bias, int dist_n, int keep,
+                                   const float* head_sinks, hipStream_t stream) {
   if (tokens <= 0) return 0;
+  if (keep < 0 || (keep > 0 && window <= 0)) MIE_FAIL("paged_attention: %d kept first keys belong beside a window", keep);
   if (dist_bias && dist_n < 1) MIE_FAIL("paged_attention: a distance bias of %d entries a head", dist_n);
   if (chunk < 0 || softcap < 0.f) MIE_FAIL("paged_attention: chunk %d, score cap %g", chunk, (double)softcap);
   if (sigmoid && has_sink) MIE_FAIL("paged_attention: a sink belongs to a softmax; the weights asked for are sigmoids");
@@ -151,7 +159,7 @@ static int paged_attention_launch(const void* q, long q_stride, const void* k_ca
 #define PA_LAUNCH(T_, NR_)                                                                                               \
   hipLaunchKernelGGL((paged_attention_kernel<T_, NR_>), grid, block, 0, stream, (const T_*)q, q_stride, (const T_*)k_cache, \
                      (const T_*)v_cache, (T_*)out, block_tables, max_blocks, token_row, positions, Hq, Hkv, D, page, scale,  \
-                     window, has_sink, sink, chunk, softcap, sigmoid, head_bias, dist_bias, dist_n)
+                     window, has_sink, sink, chunk, softcap, sigmoid, head_bias, dist_bias, dist_n, keep, head_sinks)
   if (dtype == MIE_F32 && D <= 256) PA_LAUNCH(float, 4);
   else if (dtype == MIE_F32) PA_LAUNCH(float, 16);
   else if (dtype == MIE_BF16 && D <= 256) PA_LAUNCH(bf16, 4);
@@ -167,20 +175,21 @@ MIE_EXPORT int mie_paged_attention(const void* q, long q_stride, const void* k_c
                                    const int* positions, int tokens, int Hq, int Hkv, int D, int page, float scale,
                                    int window, int has_sink, float sink, hipStream_t stream) {
   return paged_attention_launch(q, q_stride, k_cache, v_cache, out, dtype, block_tables, max_blocks, token_row, positions,
-                                tokens, Hq, Hkv, D, page, scale, window, has_sink, sink, 0, 0.f, 0, nullptr, nullptr, 0, stream);
+                                tokens, Hq, Hkv, D, page, scale, window, has_sink, sink, 0, 0.f, 0, nullptr, nullptr, 0, 0, nullptr, stream);
 }
 
 // The same with what a design may put between scores and weights: a chunk size (0: none), a cap on the scores
 // (0: none), sigmoid weights with a bias per query head (head_bias float32 [Hq] or null) instead of the softmax, a bias
 // on the score by the key's distance (dist_bias float32 [Hq, dist_n] or null: a key n positions back adds entry
-// min(n, dist_n - 1) of the head's row, after scale and cap).
+// min(n, dist_n - 1) of the head's row, after scale and cap), keep first keys beside the window (0: none), a sink per
+// query head (head_sinks float32 [Hq] or null; has_sink is then set).
 MIE_EXPORT int mie_paged_attention_scored(const void* q, long q_stride, const void* k_cache, const void* v_cache, void* out,
                                           int dtype, const int* block_tables, int max_blocks, const int* token_row,
                                           const int* positions, int tokens, int Hq, int Hkv, int D, int page, float scale,
                                           int window, int has_sink, float sink, int chunk, float softcap, int sigmoid,
-                                          const float* head_bias, const float* dist_bias, int dist_n,
-                                          hipStream_t stream) {
+                                          const float* head_bias, const float* dist_bias, int dist_n, int keep,
+                                          const float* head_sinks, hipStream_t stream) {
   return paged_attention_launch(q, q_stride, k_cache, v_cache, out, dtype, block_tables, max_blocks, token_row, positions,
                                 tokens, Hq, Hkv, D, page, scale, window, has_sink, sink, chunk, softcap, sigmoid, head_bias,
-                                dist_bias, dist_n, stream);
+                                dist_bias, dist_n, keep, head_sinks, stream);
 }

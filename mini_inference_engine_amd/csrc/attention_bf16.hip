@@ -45,7 +45,10 @@ struct ProjectionSums {
 // cap(x) = c tanh(x / c) or x itself; a chunk size n (0: none) hides the keys before floor(position / n) n.  There
 // is no maximum and no denominator: waves and splits simply add up (the merge sees maxima of 0 and one unit sum
 // a workgroup, and the kernel that joins the splits is told not to divide).  scale_log2 then carries the plain scale.
-template <int NW, bool FROM_SUMS, bool SIG = false, bool DB = false>
+// KEEP: beside the window the row sees its request's first ``keep`` keys.  The blocks that hold them come before the
+// window's in the order the splits and waves walk: index x of that order is key x up to the end of the kept blocks, key
+// x + gap behind it, gap a whole number of blocks.
+template <int NW, bool FROM_SUMS, bool SIG = false, bool DB = false, bool KEEP = false>
 __global__ void __launch_bounds__(NW * 64)
 decode_attention_kernel(const bf16* __restrict__ q, long q_stride, bf16* k_cache, bf16* v_cache,
                         bf16* __restrict__ out, float* __restrict__ o_part,
@@ -53,8 +56,9 @@ decode_attention_kernel(const bf16* __restrict__ q, long q_stride, bf16* k_cache
                         const int* __restrict__ positions, int Hq, int Hkv, int head_tiles, int page,
                         float scale_log2, int window, int partition, int num_splits, ProjectionSums proj,
                         float sink_log2, int chunk, float softcap, const float* __restrict__ head_bias,
-                        const float* __restrict__ dist_bias, int dist_n) {
+                        const float* __restrict__ dist_bias, int dist_n, int keep, const float* __restrict__ head_sinks) {
   static_assert(!(DB && (SIG || FROM_SUMS)), "the distance bias is built for the softmax over finished queries");
+  static_assert(!(KEEP && (SIG || FROM_SUMS || DB)), "kept first keys are built for the plain softmax over finished queries");
   __shared__ float s_m[NW][16], s_l[NW][16], s_M[16], s_L[16];
   __shared__ float s_o[NW][16][D + 1];
   __shared__ __align__(16) bf16 s_q[FROM_SUMS ? 16 : 1][D];
@@ -177,10 +181,18 @@ decode_attention_kernel(const bf16* __restrict__ q, long q_stride, bf16* k_cache
       sg_c3 = -L2E * hb;
     }
   }
-  const int begin = (lo & ~(BLOCK_KEYS - 1)) + s * partition;
-  const int end = begin + partition < pos + 1 ? begin + partition : pos + 1;
+  int gap = 0, kept_end = 0;
+  if constexpr (KEEP) {
+    kept_end = (keep + BLOCK_KEYS - 1) & ~(BLOCK_KEYS - 1);
+    gap = (lo & ~(BLOCK_KEYS - 1)) - kept_end;
+    gap = gap > 0 ? gap : 0;
+  }
+  const int last_x = pos - gap;                // place of the row's own key in the order the blocks are walked
+  auto key_of = [&](int x) { return !KEEP || x < kept_end ? x : x + gap; };
+  const int begin = (KEEP ? 0 : lo & ~(BLOCK_KEYS - 1)) + s * partition;
+  const int end = begin + partition < last_x + 1 ? begin + partition : last_x + 1;
 
-  if (begin > pos) {          // this split lies beyond the row's keys (uniform over the workgroup)
+  if (begin > last_x) {          // this split lies beyond the row's keys (uniform over the workgroup)
     if (num_splits > 1 && threadIdx.x < 16 && ht * 16 + (int)threadIdx.x < G)
       lse_part[((size_t)b * Hq + kvh * G + ht * 16 + threadIdx.x) * num_splits + s] = -INFINITY;
     return;
@@ -230,7 +242,7 @@ decode_attention_kernel(const bf16* __restrict__ q, long q_stride, bf16* k_cache
       for (int ks = 0; ks < KS; ++ks)
         S[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(B.a[t][ks].v, qf[ks].v, S[t], 0, 0, 0);
     }
-    const bool partial = blk + BLOCK_KEYS > pos + 1 || blk < lo;
+    const bool partial = blk + BLOCK_KEYS > pos + 1 || (blk < lo && (!KEEP || blk + BLOCK_KEYS > keep));
     if constexpr (SIG) {
       bool ok[8];
       float p[8];
@@ -276,7 +288,7 @@ decode_attention_kernel(const bf16* __restrict__ q, long q_stride, bf16* k_cache
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int key = blk + 16 * t + 4 * kb + i;
-        ok[t * 4 + i] = key >= lo && key <= pos;
+        ok[t * 4 + i] = (key >= lo || (KEEP && key < keep)) && key <= pos;
         if constexpr (DB) {
           int n = pos - key;
           n = n < 0 ? 0 : (n < dist_n ? n : dist_n - 1);            // a key after the row's own is masked
@@ -325,18 +337,18 @@ decode_attention_kernel(const bf16* __restrict__ q, long q_stride, bf16* k_cache
   constexpr int STEP = BLOCK_KEYS * NW;     // keys from one block of a wave to its next
   const int first = begin + BLOCK_KEYS * wave;
   if (AHEAD) {
-    if (window > 0 || (SIG && chunk > 0)) load_block(b0, first);  // with a window the split's start had to wait for the row's length
+    if (window > 0 || (SIG && chunk > 0)) load_block(b0, key_of(first));  // with a window the split's start had to wait for the row's length
     const int part_end = begin + partition;   // nothing is asked for beyond the split's own keys
     for (int blk = first; blk < end; blk += 2 * STEP) {
-      if (blk + STEP < part_end) load_block(b1, blk + STEP);           // in flight while block 0 is computed
-      compute(b0, blk);
-      if (blk + 2 * STEP < part_end) load_block(b0, blk + 2 * STEP);
-      if (blk + STEP < end) compute(b1, blk + STEP);
+      if (blk + STEP < part_end) load_block(b1, key_of(blk + STEP));           // in flight while block 0 is computed
+      compute(b0, key_of(blk));
+      if (blk + 2 * STEP < part_end) load_block(b0, key_of(blk + 2 * STEP));
+      if (blk + STEP < end) compute(b1, key_of(blk + STEP));
     }
   } else {
     for (int blk = first; blk < end; blk += STEP) {
-      load_block(b0, blk);
-      compute(b0, blk);
+      load_block(b0, key_of(blk));
+      compute(b0, key_of(blk));
     }
   }
 
@@ -379,7 +391,8 @@ decode_attention_kernel(const bf16* __restrict__ q, long q_stride, bf16* k_cache
     const size_t hh = (size_t)b * Hq + kvh * G + gg;
     if (num_splits == 1) {
       // a sink (sink_log2 > -inf) is one more term in the denominator; with splits the merge kernel adds it
-      out[hh * D + d] = __float2bfloat16(sum / (s_L[hc] + exp2f(sink_log2 - s_M[hc])));
+      const float sk = head_sinks ? head_sinks[kvh * G + gg] : sink_log2;
+      out[hh * D + d] = __float2bfloat16(sum / (s_L[hc] + exp2f(sk - s_M[hc])));
     } else {
       const float val = sum / s_L[hc];
       o_part[(hh * num_splits + s) * D + d] = val;
@@ -395,7 +408,7 @@ decode_attention_kernel(const bf16* __restrict__ q, long q_stride, bf16* k_cache
 // cross the per-XCD L2s, and the device-scope fences that takes cost far more than this launch.)
 __global__ void __launch_bounds__(64)
 merge_splits_kernel(const float* __restrict__ o_part, const float* __restrict__ lse_part, bf16* __restrict__ out,
-                    int num_splits, float sink_log2, int plain_sum) {
+                    int num_splits, float sink_log2, int plain_sum, const float* __restrict__ head_sinks, int Hq) {
   constexpr int DL = (D + 63) / 64;
   const size_t hh = blockIdx.x;
   const int lane = threadIdx.x;
@@ -418,6 +431,7 @@ merge_splits_kernel(const float* __restrict__ o_part, const float* __restrict__ 
       }
   };
   ask(0);
+  if (head_sinks) sink_log2 = head_sinks[hh % Hq];
   float W = 0.f;
   float M = -INFINITY;                       // the maximum over all splits first (64 a round)
   for (int s0 = 0; s0 < num_splits; s0 += 64) {
@@ -462,8 +476,11 @@ static int decode_attention_launch(const void* q, long q_stride, const void* k_c
                                    const int* positions, int rows, int Hq, int Hkv, int head_dim, int page,
                                    float scale, int window, int partition, int num_splits, float sink_log2,
                                    hipStream_t stream, bool sigmoid = false, int chunk = 0, float softcap = 0.f,
-                                   const float* head_bias = nullptr, const float* dist_bias = nullptr, int dist_n = 0) {
+                                   const float* head_bias = nullptr, const float* dist_bias = nullptr, int dist_n = 0,
+                                   int keep = 0, const float* head_sinks = nullptr) {
   if (rows <= 0) return 0;
+  if (keep < 0 || (keep > 0 && (window <= 0 || sigmoid || dist_bias)))
+    MIE_FAIL("decode_attention: %d kept first keys belong beside a window, plain softmax only", keep);
   if (dist_bias && (sigmoid || dist_n < 1)) MIE_FAIL("decode_attention: a distance bias of %d entries a head, softmax only", dist_n);
   if (chunk < 0 || softcap < 0.f) MIE_FAIL("decode_attention: chunk %d, score cap %g", chunk, (double)softcap);
   if (head_dim != D) MIE_FAIL("decode_attention: built for head_dim %d, called with %d", D, head_dim);
@@ -481,38 +498,50 @@ static int decode_attention_launch(const void* q, long q_stride, const void* k_c
   bf16* kc = (bf16*)const_cast<void*>(k_cache);
   bf16* vc = (bf16*)const_cast<void*>(v_cache);
   const bool whole = num_splits == 1 && NW_WHOLE != NW_SPLIT && (long)rows * Hkv * head_tiles < NW_WHOLE_BELOW;
-  if (dist_bias && whole)
+  if (keep > 0 && whole)
+    hipLaunchKernelGGL((decode_attention_kernel<NW_WHOLE, false, false, false, true>), grid, dim3(NW_WHOLE * 64), 0, stream, (const bf16*)q,
+                       q_stride, kc, vc, (bf16*)out, o_part, lse_part, block_tables, max_blocks, positions, Hq, Hkv, head_tiles, page,
+                       scale * 1.4426950408889634f, window, partition, num_splits, ProjectionSums{}, sink_log2, 0, 0.f,
+                       (const float*)nullptr, (const float*)nullptr, 0, keep, head_sinks);
+  else if (keep > 0)
+    hipLaunchKernelGGL((decode_attention_kernel<NW_SPLIT, false, false, false, true>), grid, dim3(NW_SPLIT * 64), 0, stream, (const bf16*)q,
+                       q_stride, kc, vc, (bf16*)out, o_part, lse_part, block_tables, max_blocks, positions, Hq, Hkv, head_tiles, page,
+                       scale * 1.4426950408889634f, window, partition, num_splits, ProjectionSums{}, sink_log2, 0, 0.f,
+                       (const float*)nullptr, (const float*)nullptr, 0, keep, head_sinks);
+  else if (dist_bias && whole)
     hipLaunchKernelGGL((decode_attention_kernel<NW_WHOLE, false, false, true>), grid, dim3(NW_WHOLE * 64), 0, stream, (const bf16*)q, q_stride,
                        kc, vc, (bf16*)out, o_part, lse_part, block_tables, max_blocks, positions, Hq, Hkv, head_tiles, page,
                        scale * 1.4426950408889634f, window, partition, num_splits, ProjectionSums{}, sink_log2, 0, 0.f,
-                       (const float*)nullptr, dist_bias, dist_n);
+                       (const float*)nullptr, dist_bias, dist_n, 0, head_sinks);
   else if (dist_bias)
     hipLaunchKernelGGL((decode_attention_kernel<NW_SPLIT, false, false, true>), grid, dim3(NW_SPLIT * 64), 0, stream, (const bf16*)q, q_stride,
                        kc, vc, (bf16*)out, o_part, lse_part, block_tables, max_blocks, positions, Hq, Hkv, head_tiles, page,
                        scale * 1.4426950408889634f, window, partition, num_splits, ProjectionSums{}, sink_log2, 0, 0.f,
-                       (const float*)nullptr, dist_bias, dist_n);
+                       (const float*)nullptr, dist_bias, dist_n, 0, head_sinks);
   else if (sigmoid && whole)
     hipLaunchKernelGGL((decode_attention_kernel<NW_WHOLE, false, true>), grid, dim3(NW_WHOLE * 64), 0, stream, (const bf16*)q, q_stride,
                        kc, vc, (bf16*)out, o_part, lse_part, block_tables, max_blocks, positions, Hq, Hkv, head_tiles, page,
-                       scale, window, partition, num_splits, ProjectionSums{}, sink_log2, chunk, softcap, head_bias, (const float*)nullptr, 0);
+                       scale, window, partition, num_splits, ProjectionSums{}, sink_log2, chunk, softcap, head_bias, (const float*)nullptr, 0, 0,
+                       head_sinks);
   else if (sigmoid)
     hipLaunchKernelGGL((decode_attention_kernel<NW_SPLIT, false, true>), grid, dim3(NW_SPLIT * 64), 0, stream, (const bf16*)q, q_stride,
                        kc, vc, (bf16*)out, o_part, lse_part, block_tables, max_blocks, positions, Hq, Hkv, head_tiles, page,
-                       scale, window, partition, num_splits, ProjectionSums{}, sink_log2, chunk, softcap, head_bias, (const float*)nullptr, 0);
+                       scale, window, partition, num_splits, ProjectionSums{}, sink_log2, chunk, softcap, head_bias, (const float*)nullptr, 0, 0,
+                       head_sinks);
   else if (whole)
     hipLaunchKernelGGL((decode_attention_kernel<NW_WHOLE, false>), grid, dim3(NW_WHOLE * 64), 0, stream, (const bf16*)q, q_stride,
                        kc, vc, (bf16*)out, o_part, lse_part, block_tables, max_blocks, positions, Hq, Hkv, head_tiles, page,
                        scale * 1.4426950408889634f, window, partition, num_splits, ProjectionSums{}, sink_log2, 0, 0.f,
-                       (const float*)nullptr, (const float*)nullptr, 0);
+                       (const float*)nullptr, (const float*)nullptr, 0, 0, head_sinks);
   else
     hipLaunchKernelGGL((decode_attention_kernel<NW_SPLIT, false>), grid, dim3(NW_SPLIT * 64), 0, stream, (const bf16*)q, q_stride,
                        kc, vc, (bf16*)out, o_part, lse_part, block_tables, max_blocks, positions, Hq, Hkv, head_tiles, page,
                        scale * 1.4426950408889634f, window, partition, num_splits, ProjectionSums{}, sink_log2, 0, 0.f,
-                       (const float*)nullptr, (const float*)nullptr, 0);
+                       (const float*)nullptr, (const float*)nullptr, 0, 0, head_sinks);
   MIE_CHECK_LAUNCH("decode_attention");
   if (num_splits > 1) {
     hipLaunchKernelGGL(merge_splits_kernel, dim3(rows * Hq), dim3(64), 0, stream, o_part, lse_part, (bf16*)out, num_splits,
-                       sink_log2, (int)sigmoid);
+                       sink_log2, (int)sigmoid, head_sinks, Hq);
     MIE_CHECK_LAUNCH("merge_splits");
   }
   return 0;
@@ -577,12 +606,12 @@ MIE_EXPORT int mie_decode_attention_from_sums(const float* part, int splits, lon
     hipLaunchKernelGGL((decode_attention_kernel<NW_WHOLE, true>), grid, dim3(NW_WHOLE * 64), 0, stream, (const bf16*)nullptr, 0L,
                        (bf16*)k_cache, (bf16*)v_cache, (bf16*)out, (float*)nullptr, (float*)nullptr, block_tables, max_blocks,
                        positions, Hq, Hkv, 1, page, scale * 1.4426950408889634f, window, partition, 1, proj, -INFINITY, 0, 0.f,
-                       (const float*)nullptr, (const float*)nullptr, 0);
+                       (const float*)nullptr, (const float*)nullptr, 0, 0, (const float*)nullptr);
   else
     hipLaunchKernelGGL((decode_attention_kernel<NW_SPLIT, true>), grid, dim3(NW_SPLIT * 64), 0, stream, (const bf16*)nullptr, 0L,
                        (bf16*)k_cache, (bf16*)v_cache, (bf16*)out, (float*)nullptr, (float*)nullptr, block_tables, max_blocks,
                        positions, Hq, Hkv, 1, page, scale * 1.4426950408889634f, window, partition, 1, proj, -INFINITY, 0, 0.f,
-                       (const float*)nullptr, (const float*)nullptr, 0);
+                       (const float*)nullptr, (const float*)nullptr, 0, 0, (const float*)nullptr);
   MIE_CHECK_LAUNCH("decode_attention_from_sums");
   return 0;
 }
@@ -659,4 +688,17 @@ MIE_EXPORT int mie_decode_attention_biased(const void* q, long q_stride, const v
   return decode_attention_launch(q, q_stride, k_cache, v_cache, out, o_part, lse_part, block_tables, max_blocks, positions,
                                  rows, Hq, Hkv, head_dim, page, scale, window, partition, num_splits, -INFINITY, stream, false,
                                  0, 0.f, nullptr, dist_bias, dist_n);
+}
+
+// The softmax over a window beside the request's first ``keep`` keys (0: none; window 0: all keys), with a sink per query head:
+// head_sinks float32 [Hq] or null, the numbers already times log2 e.  partition counts kept and window keys together: each
+// of the two starts on a block of its own.
+MIE_EXPORT int mie_decode_attention_kept(const void* q, long q_stride, const void* k_cache, const void* v_cache, void* out,
+                                         float* o_part, float* lse_part, const int* block_tables, int max_blocks,
+                                         const int* positions, int rows, int Hq, int Hkv, int head_dim, int page,
+                                         float scale, int window, int partition, int num_splits, int keep,
+                                         const float* head_sinks, hipStream_t stream) {
+  return decode_attention_launch(q, q_stride, k_cache, v_cache, out, o_part, lse_part, block_tables, max_blocks, positions,
+                                 rows, Hq, Hkv, head_dim, page, scale, window, partition, num_splits, -INFINITY, stream, false,
+                                 0, 0.f, nullptr, nullptr, 0, keep, head_sinks);
 }

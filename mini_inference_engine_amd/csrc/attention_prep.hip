@@ -7,7 +7,10 @@
 // qkv_finish: one workgroup a token.  Queries go out as [T, Hq, P], keys to k_cache [pages, Hkv, page, P], values
 // to v_cache [pages, Hkv, P, page] (transposed within a page), zeros beyond dim / vdim.  Everything is computed in
 // 32-bit from the sums and rounded once on the way out.
+// qkv_conv_finish: the same for projections that first pass a short causal convolution over time (with norms head by head,
+// halves turned, a factor on cosines and sines, values left for or mixed with another layer's).
 // head_gate:  o[t, h, :] *= sigmoid(gate[t, h]).
+// gate_heads: out[t, h vdim + d] = scale * o[t, h P + d] * sigmoid(gate[t, h vdim + d]), d < vdim.
 #include "common.hpp"
 
 enum { LAYOUT_INTERLEAVED = 0, LAYOUT_HALF = 1 };
@@ -112,6 +115,107 @@ qkv_finish_kernel(FinishArgs a) {
   }
 }
 
+// ---- projections through a short convolution
+struct ConvFinishArgs {
+  const float* sums; long ld; int col;                      // queries, keys, values side by side from column ``col`` on
+  const float* taps;            // [C, K], C = (Hq + Hkv) dim + Hkv vdim in that order
+  float* tail;                  // [slots, K - 1, C]: the row's last inputs, oldest first
+  const int* token_row; const int* row_start; const int* state_slots;
+  int K, move_tail;             // move_tail: every row is one token, and the waves move the tail on themselves
+  const float* q_norm; const float* k_norm; float eps;      // dim numbers each, or null
+  const float* inv_freq; int nf; float rot_scale;
+  const int* positions; const int* slots;
+  float* values_out; const float* mix_other; float mix;     // values as projected / (1 - mix) v + mix * other
+  void* q_out; void* k_cache; void* v_cache;
+  int Hq, Hkv, dim, vdim, P, page, C, row_floats;
+};
+
+// A workgroup a (token, share of its heads), a wave a head of queries, keys or values: its convolved numbers go into the
+// wave's own stretch of the LDS with the sum of their squares on the way, then out normed and turned.  KT: the taps (0: any
+// number).
+template <typename TO, int KT>
+__global__ void __launch_bounds__(256)
+qkv_conv_finish_kernel(ConvFinishArgs a) {
+  extern __shared__ float lds[];
+  const int t = blockIdx.x, lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
+  float* mine = lds + (size_t)wv * a.row_floats;
+  const int K = KT ? KT : a.K, keep = K - 1;
+  const int r = a.token_row[t], j = t - a.row_start[r];
+  float* __restrict__ tl = a.tail + (size_t)a.state_slots[r] * (keep > 0 ? keep : 1) * a.C;
+  const float pos = (float)a.positions[t];
+  const int slot = a.slots[t];
+  const size_t pg = slot / a.page, off = slot % a.page;
+  const int jobs = a.Hq + 2 * a.Hkv;
+  for (int job = blockIdx.y * 4 + wv; job < jobs; job += gridDim.y * 4) {
+    const bool is_q = job < a.Hq, is_v = job >= a.Hq + a.Hkv;
+    const int h = is_q ? job : is_v ? job - a.Hq - a.Hkv : job - a.Hq;
+    const int n = is_v ? a.vdim : a.dim;
+    const int c0 = is_q ? h * a.dim : is_v ? (a.Hq + a.Hkv) * a.dim + h * a.vdim : (a.Hq + h) * a.dim;
+    float ss = 0.f;
+    for (int d = lane; d < n; d += 64) {
+      const int c = c0 + d;
+      const float* __restrict__ x = a.sums + (size_t)t * a.ld + a.col + c;
+      float acc = 0.f;
+      if constexpr (KT > 0) {
+        float in[KT];
+#pragma unroll
+        for (int i = 0; i < KT; ++i) {          // tokens t - K + 1 .. t
+          const int back = KT - 1 - i;
+          const float* src = back <= j ? x - (long)back * a.ld : tl + (size_t)(keep + j - back) * a.C + c;
+          in[i] = *src;
+        }
+#pragma unroll
+        for (int i = 0; i < KT; ++i) acc = fmaf(a.taps[(size_t)c * KT + i], in[i], acc);
+        if (a.move_tail) {
+#pragma unroll
+          for (int i = 0; i < KT - 1; ++i) tl[(size_t)i * a.C + c] = in[i + 1];      // a row of one token: its inputs are the tail's and its own
+        }
+      } else {
+        for (int i = 0; i < K; ++i) {
+          const int back = K - 1 - i;
+          acc = fmaf(a.taps[(size_t)c * K + i], back <= j ? x[-(long)back * a.ld] : tl[(size_t)(keep + j - back) * a.C + c], acc);
+        }
+        if (a.move_tail)
+          for (int i = 0; i < keep; ++i) tl[(size_t)i * a.C + c] = i + 1 < keep ? tl[(size_t)(i + 1) * a.C + c] : x[0];
+      }
+      mine[d] = acc;
+      ss = fmaf(acc, acc, ss);
+    }
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");      // the wave's lanes read one another's numbers below
+    __builtin_amdgcn_wave_barrier();
+    if (is_v) {
+      TO* __restrict__ vd = (TO*)a.v_cache + (pg * a.Hkv + h) * a.P * a.page + off;
+      const size_t at = ((size_t)t * a.Hkv + h) * a.vdim;
+      for (int d = lane; d < a.P; d += 64) {
+        float v = 0.f;
+        if (d < n) {
+          v = mine[d];
+          if (a.values_out) a.values_out[at + d] = v;
+          if (a.mix_other) v = (1.0f - a.mix) * v + a.mix * a.mix_other[at + d];
+        }
+        vd[(size_t)d * a.page] = from_float<TO>(v);
+      }
+    } else {
+      const float* __restrict__ w = is_q ? a.q_norm : a.k_norm;
+      const float rms = w ? 1.0f / sqrtf(wave_sum(ss) / (float)n + a.eps) : 1.f;
+      TO* __restrict__ dst = is_q ? (TO*)a.q_out + ((size_t)t * a.Hq + h) * a.P
+                                  : (TO*)a.k_cache + ((pg * a.Hkv + h) * a.page + off) * a.P;
+      for (int i = lane; i < a.nf; i += 64) {
+        float c, s, o1, o2;
+        sincosf(pos * a.inv_freq[i], &s, &c);
+        const float x1 = w ? mine[i] * rms * w[i] : mine[i], x2 = w ? mine[i + a.nf] * rms * w[i + a.nf] : mine[i + a.nf];
+        rotate_pair(x1, x2, c * a.rot_scale, s * a.rot_scale, o1, o2);
+        dst[i] = from_float<TO>(o1);
+        dst[i + a.nf] = from_float<TO>(o2);
+      }
+      for (int d = 2 * a.nf + lane; d < a.P; d += 64)
+        dst[d] = from_float<TO>(d < n ? (w ? mine[d] * rms * w[d] : mine[d]) : 0.f);
+    }
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");      // before the next head's numbers replace these
+    __builtin_amdgcn_wave_barrier();
+  }
+}
+
 MIE_EXPORT const char* attention_prep_last_error() { return g_mie_error; }
 
 MIE_EXPORT int mie_qkv_finish(const float* sums, long ld, int q_col, int k_col, int v_col, const float* q_norm,
@@ -156,5 +260,75 @@ MIE_EXPORT int mie_head_gate(void* o, int dtype, const float* gate, long ldg, in
   else if (dtype == MIE_BF16) hipLaunchKernelGGL(head_gate_kernel<bf16>, dim3(tokens), dim3(256), 0, s, (bf16*)o, gate, ldg, H, D);
   else MIE_FAIL("head_gate: dtype code %d", dtype);
   MIE_CHECK_LAUNCH("head_gate");
+  return 0;
+}
+
+// taps [C, K] and tail [slots, max(1, K - 1), C] float32, C = (Hq + Hkv) dim + Hkv vdim channels that lie side by side in the
+// sums from column col on.  move_tail: every row of the step is one token, and the tail moves on here; else the caller moves
+// it afterwards.  values_out, mix_other float32 [tokens, Hkv vdim] or null.
+MIE_EXPORT int mie_qkv_conv_finish(const float* sums, long ld, int col, const float* taps, float* tail, const int* token_row,
+                                   const int* row_start, const int* state_slots, int K, int move_tail, const float* q_norm,
+                                   const float* k_norm, float eps, const float* inv_freq, int nf, float rot_scale,
+                                   const int* positions, const int* slots, float* values_out, const float* mix_other, float mix,
+                                   void* q_out, void* k_cache, void* v_cache, int dtype, int tokens, int Hq, int Hkv, int dim,
+                                   int vdim, int P, int page, hipStream_t s) {
+  if (tokens <= 0) return 0;
+  if (Hq <= 0 || Hkv <= 0 || dim <= 0 || vdim <= 0 || P < dim || P < vdim || page <= 0 || P > 1024)
+    MIE_FAIL("qkv_conv_finish: %d / %d heads of %d (values %d) in %d (at most 1024), page %d", Hq, Hkv, dim, vdim, P, page);
+  if (2 * nf > dim || nf < 0 || (nf > 0 && !inv_freq)) MIE_FAIL("qkv_conv_finish: %d turned pairs in heads of %d", nf, dim);
+  if (K < 1 || !taps || !tail || !token_row || !row_start || !state_slots) MIE_FAIL("qkv_conv_finish: %d taps and their operands", K);
+  const int C = (Hq + Hkv) * dim + Hkv * vdim;
+  if (ld < (long)col + C) MIE_FAIL("qkv_conv_finish: %d channels from column %d in rows of %ld", C, col, ld);
+  const int row_floats = (dim > vdim ? dim : vdim);
+  ConvFinishArgs a{sums, ld, col, taps, tail, token_row, row_start, state_slots, K, move_tail, q_norm, k_norm, eps, inv_freq, nf,
+                   rot_scale, positions, slots, values_out, mix_other, mix, q_out, k_cache, v_cache, Hq, Hkv, dim, vdim, P, page, C,
+                   row_floats};
+  const size_t lds = (size_t)4 * row_floats * sizeof(float);
+  int parts = (Hq + 2 * Hkv + 3) / 4;
+  const int most = tokens >= 1024 ? 4 : 16;
+  parts = parts < most ? parts : most;
+#define QCF(T_, K_) hipLaunchKernelGGL((qkv_conv_finish_kernel<T_, K_>), dim3(tokens, parts), dim3(256), lds, s, a)
+#define QCF_K(T_)              \
+  switch (K) {                 \
+    case 2: QCF(T_, 2); break; \
+    case 3: QCF(T_, 3); break; \
+    case 4: QCF(T_, 4); break; \
+    default: QCF(T_, 0);       \
+  }
+  if (dtype == MIE_F32) { QCF_K(float) }
+  else if (dtype == MIE_BF16) { QCF_K(bf16) }
+  else MIE_FAIL("qkv_conv_finish: dtype code %d", dtype);
+#undef QCF_K
+#undef QCF
+  MIE_CHECK_LAUNCH("qkv_conv_finish");
+  return 0;
+}
+
+template <typename T>
+__global__ void __launch_bounds__(256)
+gate_heads_kernel(const T* __restrict__ o, const float* __restrict__ gate, long ldg, T* __restrict__ out, long ldo, int H, int dv,
+                  int P, float scale) {
+  const int t = blockIdx.x;
+  const T* __restrict__ row = o + (size_t)t * H * P;
+  for (int e = blockIdx.y * blockDim.x + threadIdx.x; e < H * dv; e += gridDim.y * blockDim.x) {
+    const int h = e / dv;
+    out[(size_t)t * ldo + e] = from_float<T>(scale * to_float(row[h * P + e - h * dv]) * mie_sigmoid(gate[(size_t)t * ldg + e]));
+  }
+}
+
+// gate points at the first gate column; rows of gate are ldg floats apart, rows of out ldo numbers
+MIE_EXPORT int mie_gate_heads(const void* o, int dtype, const float* gate, long ldg, void* out, long ldo, int tokens, int H, int dv,
+                              int P, float scale, hipStream_t s) {
+  if (tokens <= 0) return 0;
+  if (H <= 0 || dv <= 0 || P < dv || ldg < (long)H * dv || ldo < (long)H * dv)
+    MIE_FAIL("gate_heads: %d heads of %d in %d, gate rows %ld apart, output rows %ld", H, dv, P, ldg, ldo);
+  int by = (H * dv + 1023) / 1024;
+  by = by > 16 ? 16 : by;
+  if (dtype == MIE_F32)
+    hipLaunchKernelGGL(gate_heads_kernel<float>, dim3(tokens, by), dim3(256), 0, s, (const float*)o, gate, ldg, (float*)out, ldo, H, dv, P, scale);
+  else if (dtype == MIE_BF16)
+    hipLaunchKernelGGL(gate_heads_kernel<bf16>, dim3(tokens, by), dim3(256), 0, s, (const bf16*)o, gate, ldg, (bf16*)out, ldo, H, dv, P, scale);
+  else MIE_FAIL("gate_heads: dtype code %d", dtype);
+  MIE_CHECK_LAUNCH("gate_heads");
   return 0;
 }

@@ -250,6 +250,50 @@ clamped_glu_kernel(const float* __restrict__ in, long ld_in, TO* __restrict__ ou
   }
 }
 
+// the same from bfloat16 sums whose gate and up halves start on 16 bytes, eight values a thread and a load
+__global__ void __launch_bounds__(256)
+clamped_glu_bf16x8_kernel(const bf16* __restrict__ gu, long ld_in, bf16* __restrict__ out, long ld_out, int rows, int inter,
+                          float limit, float alpha, float shift) {
+  const int per_row = inter >> 3;
+  const size_t total = (size_t)rows * per_row;
+  const float slope = alpha * -1.4426950408889634f;
+  for (size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x; idx < total; idx += (size_t)gridDim.x * blockDim.x) {
+    const size_t r = idx / per_row, i = (idx - r * per_row) << 3;
+    const uint4 g4 = *reinterpret_cast<const uint4*>(gu + r * ld_in + i);
+    const uint4 u4 = *reinterpret_cast<const uint4*>(gu + r * ld_in + inter + i);
+    const uint32_t gw[4] = {g4.x, g4.y, g4.z, g4.w}, uw[4] = {u4.x, u4.y, u4.z, u4.w};
+    uint32_t ow[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      uint32_t word = 0;
+#pragma unroll
+      for (int e = 0; e < 2; ++e) {
+        const float g = fminf(__uint_as_float(e ? gw[j] & 0xFFFF0000u : gw[j] << 16), limit);
+        const float u = fminf(fmaxf(__uint_as_float(e ? uw[j] & 0xFFFF0000u : uw[j] << 16), -limit), limit);
+        const float s = __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(g * slope));
+        word |= (uint32_t)__builtin_bit_cast(uint16_t, __float2bfloat16(g * s * (u + shift))) << (16 * e);
+      }
+      ow[j] = word;
+    }
+    *reinterpret_cast<uint4*>(out + r * ld_out + i) = make_uint4(ow[0], ow[1], ow[2], ow[3]);
+  }
+}
+
+// gu bfloat16 [rows, 2 inner] (gate values, then up values) -> out bfloat16 [rows, inner]
+MIE_EXPORT int mie_clamped_glu_bf16(const void* gu, long ld_in, void* out, long ld_out, int rows, int inner, float limit, float alpha,
+                                    float shift, hipStream_t s) {
+  if (rows <= 0 || inner <= 0) return 0;
+  if ((inner & 7) || (ld_in & 7) || (ld_out & 7) || (((uintptr_t)gu | (uintptr_t)out) & 15) || ld_in < 2L * inner || ld_out < inner)
+    MIE_FAIL("clamped_glu_bf16: inner size %d, leading dims %ld, %ld (multiples of 8, 16-byte aligned)", inner, ld_in, ld_out);
+  if (!(limit > 0.f)) MIE_FAIL("clamped_glu_bf16: limit %g", (double)limit);
+  long blocks = ((long)rows * (inner / 8) + 255) / 256;
+  if (blocks > 16384) blocks = 16384;
+  hipLaunchKernelGGL(clamped_glu_bf16x8_kernel, dim3((unsigned)blocks), dim3(256), 0, s, (const bf16*)gu, ld_in, (bf16*)out, ld_out,
+                     rows, inner, limit, alpha, shift);
+  MIE_CHECK_LAUNCH("clamped_glu_bf16");
+  return 0;
+}
+
 MIE_EXPORT int mie_act_store(const float* in, long ld_in, void* out, long ld_out, int out_dtype, int rows, int n, int act,
                              hipStream_t s) {
   if (rows <= 0 || n <= 0) return 0;

@@ -73,9 +73,10 @@ template <int SLOTS, int IT> struct RingStart {
   }
 };
 
-enum { EPI_STORE_BF16 = 0, EPI_STORE_F32 = 1, EPI_ADD = 2, EPI_SWIGLU = 3, EPI_ROPE = 4, EPI_GEGLU = 5 };
-// the gated epilogues differ in the gate's function only: silu (SWIGLU) or the tanh form of gelu (GEGLU)
-#define EPI_GATED(E) ((E) == EPI_SWIGLU || (E) == EPI_GEGLU)
+enum { EPI_STORE_BF16 = 0, EPI_STORE_F32 = 1, EPI_ADD = 2, EPI_SWIGLU = 3, EPI_ROPE = 4, EPI_GEGLU = 5, EPI_CLAMPGLU = 6 };
+// the gated epilogues differ in the function only: silu(g) u (SWIGLU), the tanh form of gelu(g) u (GEGLU), or, with g at most
+// a limit and u within plus and minus that limit, g sigmoid(alpha g) (u + shift) (CLAMPGLU)
+#define EPI_GATED(E) ((E) == EPI_SWIGLU || (E) == EPI_GEGLU || (E) == EPI_CLAMPGLU)
 
 // What the rotary epilogue needs beside the product: W is the fused q/k/v projection; the workgroup owns
 // columns j0 .. j0 + 7 and j0 + D/2 .. j0 + D/2 + 7 of one head, i.e. 8 rotary pairs.
@@ -105,6 +106,7 @@ struct NormArgs {
   int ss_tiles;
   float inv_width, eps;
   const int* rows;           // others: optional gather of X's (and ss_in's) rows, int32 [M]
+  float glu_limit, glu_alpha, glu_shift;     // CLAMPGLU's constants (with or without a fused norm)
 };
 
 // Which weight row column c (0 .. 15) of tile `tile` multiplies, and whether it exists.
@@ -321,8 +323,13 @@ skinny_gemm_kernel(const bf16* __restrict__ X, long ldx, const bf16* __restrict_
   } else if (EPI == EPI_STORE_F32) {
     ((float*)outv)[(size_t)m * ldo + n] = mine_v;
   } else if (c < 8) {                        // gated: mine = gate, other = up
-    const float a = EPI == EPI_GEGLU ? mie_gelu_tanh(mine_v) : mine_v / (1.0f + expf(-mine_v));
-    ((bf16*)outv)[(size_t)m * ldo + n] = __float2bfloat16(a * other);
+    if (EPI == EPI_CLAMPGLU) {
+      const float g = fminf(mine_v, nf.glu_limit), u = fminf(fmaxf(other, -nf.glu_limit), nf.glu_limit);
+      ((bf16*)outv)[(size_t)m * ldo + n] = __float2bfloat16(g * mie_sigmoid(nf.glu_alpha * g) * (u + nf.glu_shift));
+    } else {
+      const float a = EPI == EPI_GEGLU ? mie_gelu_tanh(mine_v) : mine_v / (1.0f + expf(-mine_v));
+      ((bf16*)outv)[(size_t)m * ldo + n] = __float2bfloat16(a * other);
+    }
   }
 }
 
@@ -359,6 +366,7 @@ static int launch_epi(int epi, dim3 grid, hipStream_t s, const bf16* X, long ldx
     case EPI_ADD: SG_LAUNCH(EPI_ADD); break;
     case EPI_SWIGLU: SG_LAUNCH(EPI_SWIGLU); break;
     case EPI_GEGLU: SG_LAUNCH(EPI_GEGLU); break;
+    case EPI_CLAMPGLU: SG_LAUNCH(EPI_CLAMPGLU); break;
     case EPI_ROPE: SG_LAUNCH(EPI_ROPE); break;
     default: MIE_FAIL("skinny_gemm: epilogue code %d", epi);
   }
@@ -386,14 +394,12 @@ static int slots_for(int tiles) {
 }
 
 static int launch_rows(int tiles, int epi, hipStream_t s, const bf16* X, long ldx, const bf16* W, long ldw, void* out,
-                       long ldo, int M, int N, int K, int up_offset, const RopeArgs& rope, const NormArgs* nf) {
+                       long ldo, int M, int N, int K, int up_offset, const RopeArgs& rope, const NormArgs& n, bool fused) {
   dim3 grid(tiles);
-  NormArgs none = {};
-  const NormArgs& n = nf ? *nf : none;
   if (slots_for(tiles) == 3)
-    return nf ? launch_epi<true, 3>(epi, grid, s, X, ldx, W, ldw, out, ldo, M, N, K, up_offset, rope, n)
-              : launch_epi<false, 3>(epi, grid, s, X, ldx, W, ldw, out, ldo, M, N, K, up_offset, rope, n);
-  return nf ? launch_epi<true, 4>(epi, grid, s, X, ldx, W, ldw, out, ldo, M, N, K, up_offset, rope, n)
+    return fused ? launch_epi<true, 3>(epi, grid, s, X, ldx, W, ldw, out, ldo, M, N, K, up_offset, rope, n)
+                 : launch_epi<false, 3>(epi, grid, s, X, ldx, W, ldw, out, ldo, M, N, K, up_offset, rope, n);
+  return fused ? launch_epi<true, 4>(epi, grid, s, X, ldx, W, ldw, out, ldo, M, N, K, up_offset, rope, n)
             : launch_epi<false, 4>(epi, grid, s, X, ldx, W, ldw, out, ldo, M, N, K, up_offset, rope, n);
 }
 
@@ -435,12 +441,28 @@ MIE_EXPORT int mie_skinny_gemm(const void* X, long ldx, const void* W, long ldw,
   if (check_operands("skinny_gemm", X, ldx, W, ldw, M, K)) return -1;
   if (ldo < N) MIE_FAIL("skinny_gemm: output leading dim %ld < %d", ldo, N);
   RopeArgs none = {};
-  NormArgs nf;
+  NormArgs nf = {};
   const bool fused = next_g || ss_in;
   if (fused && fill_norm_args(nf, epi, next_g, next_g_f32, x_next, ldx_next, ss_out, ss_in, ss_tiles, K, eps, rows, N)) return -1;
   if (!fused && rows) MIE_FAIL("skinny_gemm: a row gather comes with the fused norm only");
   return launch_rows(EPI_GATED(epi) ? (N + 7) / 8 : (N + 15) / 16, epi, s, (const bf16*)X, ldx, (const bf16*)W, ldw, out, ldo, M, N, K, N, none,
-                     fused ? &nf : nullptr);
+                     nf, fused);
+}
+
+// g sigmoid(alpha g) (u + shift) with g = min(gate, limit), u = clamp(up, -limit, limit); W = [gate rows (N of them); up rows],
+// N the intermediate size, out bfloat16 [M, ldo].  With ss_in: X is a fused-norm producer's x_next (see above).
+MIE_EXPORT int mie_skinny_clamped_glu(const void* X, long ldx, const void* W, long ldw, void* out, long ldo, int M, int N, int K,
+                                      float limit, float alpha, float shift, const float* ss_in, int ss_tiles, float eps,
+                                      const int* rows, hipStream_t s) {
+  if (M <= 0 || N <= 0) return 0;
+  if (check_operands("skinny_clamped_glu", X, ldx, W, ldw, M, K)) return -1;
+  if (ldo < N || !(limit > 0.f)) MIE_FAIL("skinny_clamped_glu: output leading dim %ld < %d, limit %g", ldo, N, (double)limit);
+  if (!ss_in && rows) MIE_FAIL("skinny_clamped_glu: a row gather comes with the fused norm only");
+  RopeArgs none = {};
+  NormArgs nf = {};
+  if (ss_in && fill_norm_args(nf, EPI_CLAMPGLU, nullptr, 0, nullptr, 0, nullptr, ss_in, ss_tiles, K, eps, rows, N)) return -1;
+  nf.glu_limit = limit; nf.glu_alpha = alpha; nf.glu_shift = shift;
+  return launch_rows((N + 7) / 8, EPI_CLAMPGLU, s, (const bf16*)X, ldx, (const bf16*)W, ldw, out, ldo, M, N, K, N, none, nf, ss_in != nullptr);
 }
 
 // The fused q/k/v projection of single-token rows with what follows it: W [(Hq + 2 Hkv) D, K]; rotary
@@ -460,8 +482,8 @@ MIE_EXPORT int mie_skinny_qkv_rope(const void* X, long ldx, const void* W, long 
   if (ldq < (long)Hq * D) MIE_FAIL("skinny_qkv_rope: q leading dim %ld < %d", ldq, Hq * D);
   RopeArgs rope = {positions, cos_t, sin_t, slots, (bf16*)k_cache, (bf16*)v_cache, Hq, Hkv, D, page};
   const int heads = Hq + 2 * Hkv;
-  NormArgs nf;
+  NormArgs nf = {};
   if (ss_in && fill_norm_args(nf, EPI_ROPE, nullptr, 0, nullptr, 0, nullptr, ss_in, ss_tiles, K, eps, nullptr, heads * D)) return -1;
   return launch_rows(heads * (D / 16), EPI_ROPE, s, (const bf16*)X, ldx, (const bf16*)W, ldw, q_out, ldq, M, heads * D, K,
-                     D / 2, rope, ss_in ? &nf : nullptr);
+                     D / 2, rope, nf, ss_in != nullptr);
 }

@@ -35,6 +35,9 @@
 //
 // DB: a bias on the softmax's scores by the key's distance, from a table a head (its last entry for everything
 // further back), added after the scale; the running maximum then lives in units of log2 e of the biased score.
+//
+// KEEP: beside the window a query sees its request's first ``keep`` keys.  The steps that hold them come before the
+// window's: place x in the order of the steps is key x up to the end of the kept steps, key x + gap behind it.
 typedef float f32x16 __attribute__((ext_vector_type(16)));
 struct __attribute__((packed, aligned(4))) Run4 { float a, b, c, d; };      // four table entries in a row, 4-byte aligned
 
@@ -78,15 +81,17 @@ __device__ __forceinline__ float pair_sum(float x) {
 // KS = 2: the waves form two halves that take the even and the odd 64-key blocks of the same queries (a step
 // brings 128 keys in, each half computes its 64) and join their results at the end: half the blocks a wave
 // for rows too short to give every SIMD two waves otherwise.
-template <int PF_WAVES, int KS, bool SIG, bool DB = false>
+template <int PF_WAVES, int KS, bool SIG, bool DB = false, bool KEEP = false>
 __global__ void __launch_bounds__(PF_WAVES * 64)
 prefill_attention_kernel(const bf16* __restrict__ q, long q_stride, const bf16* __restrict__ k_cache,
                          const bf16* __restrict__ v_cache, bf16* __restrict__ out,
                          const int* __restrict__ block_tables, int max_blocks, const int* __restrict__ row_start,
                          const int* __restrict__ row_position, int first_row, int Hq, int Hkv, int waves_h,
                          int page, float scale_log2, int window, float sink_log2, int chunk, float softcap,
-                         const float* __restrict__ head_bias, const float* __restrict__ dist_bias, int dist_n) {
+                         const float* __restrict__ head_bias, const float* __restrict__ dist_bias, int dist_n, int keep,
+                         const float* __restrict__ head_sinks) {
   static_assert(!(SIG && DB), "the distance bias is built for the softmax");
+  static_assert(!(KEEP && (SIG || DB)), "kept first keys are built for the plain softmax");
   extern __shared__ __align__(16) unsigned char pf_lds[];
   constexpr int PF_THREADS = PF_WAVES * 64;
   constexpr int SUB_WAVES = PF_WAVES / KS;                   // waves of one half
@@ -192,7 +197,15 @@ prefill_attention_kernel(const bf16* __restrict__ q, long q_stride, const bf16* 
         sg_c3 = -L2E * hb;
       }
     }
-    const int blk0 = kmin & ~(PF_BK - 1);
+    int gap = 0, kept_end = 0;
+    if constexpr (KEEP) {
+      kept_end = (keep + FK - 1) / FK * FK;
+      gap = (kmin & ~(PF_BK - 1)) - kept_end;
+      gap = gap > 0 ? gap : 0;
+    }
+    const int last_x = kmax - gap;                             // place of the last key in the order of the steps
+    auto key_of = [&](int x) { return !KEEP || x < kept_end ? x : x + gap; };
+    const int blk0 = KEEP ? 0 : kmin & ~(PF_BK - 1);
     const int last_blk = kmax & ~(PF_BK - 1);
     // DB: the head's row of the distance table (its entries already times log2 e); scores leave the bias step scaled
     const float* __restrict__ db_row = DB ? dist_bias + (size_t)head * dist_n : nullptr;
@@ -220,8 +233,12 @@ prefill_attention_kernel(const bf16* __restrict__ q, long q_stride, const bf16* 
     // pages of a power of two (the usual 16): a key's page by a shift (the same for every lane)
     const int page_shift = (page & (page - 1)) == 0 ? __builtin_ctz(page) : -1;
     auto lookup = [&](Where& Wh, int blk) {            // blocks are looked up in order, 64 keys apart
+      blk = key_of(blk);
       blk = blk < last_blk ? blk : last_blk;           // beyond the last block: the last one again
-      {
+      if constexpr (KEEP) {
+        walk_idx = page_shift >= 0 ? blk >> page_shift : blk / page;
+        walk_start = walk_idx * page;
+      } else {
         const int d = blk - walk_start;
         int adv = 0;
         if (page_shift >= 0) {
@@ -356,8 +373,8 @@ prefill_attention_kernel(const bf16* __restrict__ q, long q_stride, const bf16* 
         }
       }
       // every query of the tile sees every key of the block (uniform over the wave)
-      const bool whole = blk + PF_BK - 1 <= tile_first && (window <= 0 || blk >= tile_last - window + 1) &&
-                         (!SIG || blk >= tile_lo);
+      const bool whole = blk + PF_BK - 1 <= tile_first &&
+                         (window <= 0 || blk >= tile_last - window + 1 || (KEEP && blk + PF_BK <= keep)) && (!SIG || blk >= tile_lo);
       if constexpr (DB) {
 #pragma unroll
         for (int u = 0; u < 2; ++u)
@@ -430,7 +447,7 @@ prefill_attention_kernel(const bf16* __restrict__ q, long q_stride, const bf16* 
 #pragma unroll
           for (int i = 0; i < 16; ++i) {
             const int key = blk + 32 * u + 8 * (i >> 2) + 4 * g + (i & 3);
-            const bool ok = key >= lo && key <= hi;
+            const bool ok = (key >= lo || (KEEP && key < keep)) && key <= hi;
             S[u][i] = ok ? S[u][i] : -INFINITY;
             mx = max_nn(mx, S[u][i]);
           }
@@ -484,27 +501,27 @@ prefill_attention_kernel(const bf16* __restrict__ q, long q_stride, const bf16* 
     fetch(pb_, wh_);                                   // step 1 (clamped into the row if there is none)
     lookup(wh_, blk0 + 2 * FK);
     __syncthreads();                                   // the previous stretch is done with the buffers
-    stash(pa, 0, blk0);
+    stash(pa, 0, key_of(blk0));
     __syncthreads();
     const int mine_off = wk * PF_BK;                   // this wave's block within a step
-    auto mine = [&](int blk) { return blk <= wave_kmax && blk + PF_BK > wave_kmin; };
-    for (int blk = blk0; blk <= kmax; blk += 2 * FK) {         // every condition is uniform over the workgroup
+    auto mine = [&](int blk) { return blk <= wave_kmax && (blk + PF_BK > wave_kmin || (KEEP && blk < keep)); };
+    for (int blk = blk0; blk <= last_x; blk += 2 * FK) {       // every condition is uniform over the workgroup
       // step blk from set 0; pb_ holds step blk + FK; pa is free for step blk + 2 FK
-      if (blk + 2 * FK <= kmax) {
+      if (blk + 2 * FK <= last_x) {
         fetch(pa, wh_);
         lookup(wh_, blk + 3 * FK);
       }
-      if (mine(blk + mine_off)) compute(0, blk + mine_off);
-      if (blk + FK > kmax) break;
-      stash(pb_, 1, blk + FK);
+      if (mine(key_of(blk) + mine_off)) compute(0, key_of(blk) + mine_off);
+      if (blk + FK > last_x) break;
+      stash(pb_, 1, key_of(blk + FK));
       __syncthreads();
       // step blk + FK from set 1; pa holds step blk + 2 FK; pb_ is free for step blk + 3 FK
-      if (blk + 3 * FK <= kmax) {
+      if (blk + 3 * FK <= last_x) {
         fetch(pb_, wh_);
         lookup(wh_, blk + 4 * FK);
       }
-      if (mine(blk + FK + mine_off)) compute(1, blk + FK + mine_off);
-      if (blk + 2 * FK <= kmax) stash(pa, 0, blk + 2 * FK);
+      if (mine(key_of(blk + FK) + mine_off)) compute(1, key_of(blk + FK) + mine_off);
+      if (blk + 2 * FK <= last_x) stash(pa, 0, key_of(blk + 2 * FK));
       __syncthreads();
     }
 
@@ -549,7 +566,7 @@ prefill_attention_kernel(const bf16* __restrict__ q, long q_stride, const bf16* 
     const float total = pair_sum(l);
     if (q_ok && wk == 0) {
       // a sink (sink_log2 > -inf) is one more term in the denominator; m is finite: a query sees its own key
-      const float inv = SIG ? 1.0f : 1.0f / (total + fast_exp2(sink_log2 - m));
+      const float inv = SIG ? 1.0f : 1.0f / (total + fast_exp2((head_sinks ? head_sinks[head] : sink_log2) - m));
       bf16* op = out + ((size_t)qtok * Hq + head) * D + 4 * g;
 #pragma unroll
       for (int dt = 0; dt < DT32; ++dt)
@@ -576,8 +593,11 @@ static int prefill_attention_launch(const void* q, long q_stride, const void* k_
                                     const int* row_position, int first_row, int rows, int max_row_tokens, int Hq,
                                     int Hkv, int head_dim, int page, float scale, int window, float sink_log2,
                                     hipStream_t stream, bool sigmoid = false, int chunk = 0, float softcap = 0.f,
-                                    const float* head_bias = nullptr, const float* dist_bias = nullptr, int dist_n = 0) {
+                                    const float* head_bias = nullptr, const float* dist_bias = nullptr, int dist_n = 0,
+                                    int keep = 0, const float* head_sinks = nullptr) {
   if (rows <= 0 || max_row_tokens <= 0) return 0;
+  if (keep < 0 || (keep > 0 && (window <= 0 || sigmoid || dist_bias)))
+    MIE_FAIL("prefill_attention: %d kept first keys belong beside a window, plain softmax only", keep);
   if (dist_bias && (sigmoid || dist_n < 1)) MIE_FAIL("prefill_attention: a distance bias of %d entries a head, softmax only", dist_n);
   if (chunk < 0 || softcap < 0.f) MIE_FAIL("prefill_attention: chunk %d, score cap %g", chunk, (double)softcap);
   if (head_dim != D) MIE_FAIL("prefill_attention: built for head_dim %d, called with %d", D, head_dim);
@@ -623,9 +643,9 @@ static int prefill_attention_launch(const void* q, long q_stride, const void* k_
   if (grid.y > 65535 || grid.z > 65535) MIE_FAIL("prefill_attention: grid too large (%d rows)", rows);
   const float scale_log2 = sigmoid ? scale : scale * 1.4426950408889634f;      // the sigmoid kernels fold their own constants
   // more LDS than a kernel gets by default is asked for once per kernel and device
-  static bool lds_allowed[9][64] = {};
+  static bool lds_allowed[12][64] = {};
   auto launch = [&](auto kernel, int waves, int lds_bytes) -> int {
-    const int which = kind + (sigmoid ? 3 : 0) + (dist_bias ? 6 : 0);
+    const int which = kind + (sigmoid ? 3 : 0) + (dist_bias ? 6 : 0) + (keep > 0 ? 9 : 0);
     if (lds_bytes > 64 * 1024 && !lds_allowed[which][dev]) {
       hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, lds_bytes);
       if (e != hipSuccess) MIE_FAIL("prefill_attention: %d bytes of LDS refused: %s", lds_bytes, hipGetErrorString(e));
@@ -633,20 +653,24 @@ static int prefill_attention_launch(const void* q, long q_stride, const void* k_
     }
     hipLaunchKernelGGL(kernel, grid, dim3(waves * 64), lds_bytes, stream, (const bf16*)q, q_stride, (const bf16*)k_cache,
                        (const bf16*)v_cache, (bf16*)out, block_tables, max_blocks, row_start, row_position, first_row, Hq, Hkv,
-                       waves_h, page, scale_log2, window, sink_log2, chunk, softcap, head_bias, dist_bias, dist_n);
+                       waves_h, page, scale_log2, window, sink_log2, chunk, softcap, head_bias, dist_bias, dist_n, keep,
+                       head_sinks);
     return 0;
   };
   int rc = 0;
-  const bool plain = !sigmoid && !dist_bias;
+  const bool plain = !sigmoid && !dist_bias && keep == 0;
   if constexpr (PF_MAX_WAVES == 8) {
     if (kind == EIGHT_QUERIES && dist_bias) rc = launch(prefill_attention_kernel<8, 1, false, true>, 8, 2 * PF_BUF);
     if (kind == EIGHT_KEYS && dist_bias) rc = launch(prefill_attention_kernel<8, 2, false, true>, 8, 4 * PF_BUF);
     if (kind == EIGHT_QUERIES && plain) rc = launch(prefill_attention_kernel<8, 1, false>, 8, 2 * PF_BUF);
     if (kind == EIGHT_KEYS && plain) rc = launch(prefill_attention_kernel<8, 2, false>, 8, 4 * PF_BUF);
+    if (kind == EIGHT_QUERIES && keep > 0) rc = launch(prefill_attention_kernel<8, 1, false, false, true>, 8, 2 * PF_BUF);
+    if (kind == EIGHT_KEYS && keep > 0) rc = launch(prefill_attention_kernel<8, 2, false, false, true>, 8, 4 * PF_BUF);
     if (kind == EIGHT_QUERIES && sigmoid) rc = launch(prefill_attention_kernel<8, 1, true>, 8, 2 * PF_BUF);
     if (kind == EIGHT_KEYS && sigmoid) rc = launch(prefill_attention_kernel<8, 2, true>, 8, 4 * PF_BUF);
   }
   if (kind == FOUR && dist_bias) rc = launch(prefill_attention_kernel<4, 1, false, true>, 4, 2 * PF_BUF);
+  if (kind == FOUR && keep > 0) rc = launch(prefill_attention_kernel<4, 1, false, false, true>, 4, 2 * PF_BUF);
   if (kind == FOUR && plain) rc = launch(prefill_attention_kernel<4, 1, false>, 4, 2 * PF_BUF);
   if (kind == FOUR && sigmoid) rc = launch(prefill_attention_kernel<4, 1, true>, 4, 2 * PF_BUF);
   if (rc) return rc;
@@ -697,4 +721,16 @@ MIE_EXPORT int mie_prefill_attention_biased(const void* q, long q_stride, const 
   return prefill_attention_launch(q, q_stride, k_cache, v_cache, out, block_tables, max_blocks, row_start, row_position,
                                   first_row, rows, max_row_tokens, Hq, Hkv, head_dim, page, scale, window, -INFINITY, stream,
                                   false, 0, 0.f, nullptr, dist_bias, dist_n);
+}
+
+// The softmax over a window beside the request's first ``keep`` keys (0: none; window 0: all keys), with a sink per query head:
+// head_sinks float32 [Hq] or null, the numbers already times log2 e.
+MIE_EXPORT int mie_prefill_attention_kept(const void* q, long q_stride, const void* k_cache, const void* v_cache, void* out,
+                                          const int* block_tables, int max_blocks, const int* row_start,
+                                          const int* row_position, int first_row, int rows, int max_row_tokens, int Hq,
+                                          int Hkv, int head_dim, int page, float scale, int window, int keep,
+                                          const float* head_sinks, hipStream_t stream) {
+  return prefill_attention_launch(q, q_stride, k_cache, v_cache, out, block_tables, max_blocks, row_start, row_position,
+                                  first_row, rows, max_row_tokens, Hq, Hkv, head_dim, page, scale, window, -INFINITY, stream,
+                                  false, 0, 0.f, nullptr, nullptr, 0, keep, head_sinks);
 }

@@ -64,6 +64,61 @@ conv_tail_update_kernel(const float* __restrict__ h, float* __restrict__ tail, c
   }
 }
 
+// short_conv: u[t, c] = act(bias[c] + sum_k taps[c, k] x[t - (K - 1 - k), c]); inputs before the row's first token come from
+// tail[slot].  move_tail (every row is one token): the thread moves its channel of the tail on; else the tail is only
+// read here and conv_tail_move, launched after it, moves it.
+template <int KT>
+__global__ void __launch_bounds__(256)
+short_conv_kernel(const float* __restrict__ x, long ldx, const float* __restrict__ taps, const float* __restrict__ bias,
+                  float* __restrict__ tail, const int* __restrict__ token_row, const int* __restrict__ row_start,
+                  const int* __restrict__ slots, float* __restrict__ u, int C, int K_any, int act, int move_tail) {
+  const int K = KT ? KT : K_any, keep = K - 1;
+  const int t = blockIdx.x;
+  const int r = token_row[t], j = t - row_start[r];
+  float* __restrict__ tl = tail + (size_t)slots[r] * (keep > 0 ? keep : 1) * C;
+  for (int c = blockIdx.y * blockDim.x + threadIdx.x; c < C; c += gridDim.y * blockDim.x) {
+    const float* __restrict__ xc = x + (size_t)t * ldx + c;
+    float acc = bias ? bias[c] : 0.f;
+    if constexpr (KT > 0) {
+      float in[KT];
+#pragma unroll
+      for (int i = 0; i < KT; ++i) {
+        const int back = KT - 1 - i;
+        const float* src = back <= j ? xc - (long)back * ldx : tl + (size_t)(keep + j - back) * C + c;
+        in[i] = *src;
+      }
+#pragma unroll
+      for (int i = 0; i < KT; ++i) acc = fmaf(taps[(size_t)c * KT + i], in[i], acc);
+      if (move_tail) {
+#pragma unroll
+        for (int i = 0; i < KT - 1; ++i) tl[(size_t)i * C + c] = in[i + 1];
+      }
+    } else {
+      for (int i = 0; i < K; ++i) {
+        const int back = K - 1 - i;
+        acc = fmaf(taps[(size_t)c * K + i], back <= j ? xc[-(long)back * ldx] : tl[(size_t)(keep + j - back) * C + c], acc);
+      }
+      if (move_tail)
+        for (int i = 0; i < keep; ++i) tl[(size_t)i * C + c] = i + 1 < keep ? tl[(size_t)(i + 1) * C + c] : xc[0];
+    }
+    u[(size_t)t * C + c] = mie_act(acc, act);
+  }
+}
+
+// the row's last K - 1 inputs (old tail, then this step's x), oldest first, into tail[slot]; a thread a (row, channel)
+__global__ void __launch_bounds__(256)
+conv_tail_move_kernel(const float* __restrict__ x, long ldx, float* __restrict__ tail, const int* __restrict__ row_start,
+                      const int* __restrict__ slots, int C, int K) {
+  const int r = blockIdx.x, c = blockIdx.y * blockDim.x + threadIdx.x;
+  if (c >= C) return;
+  const int a0 = row_start[r], n = row_start[r + 1] - a0, keep = K - 1;
+  float* tl = tail + (size_t)slots[r] * keep * C;
+  for (int i = 0; i < keep; ++i) {
+    const int src = n + i;                     // place in the joined sequence of keep + n inputs
+    tl[(size_t)i * C + c] = src < keep ? tl[(size_t)src * C + c] : x[(size_t)(a0 + src - keep) * ldx + c];
+  }
+}
+
 template <typename TO>
 __global__ void __launch_bounds__(256)
 rglru_scan_kernel(const float* __restrict__ u, const float* __restrict__ gates, const float* __restrict__ lam,
@@ -250,5 +305,39 @@ MIE_EXPORT int mie_residual_conv(const float* h, const float* taps, float* tail,
     hipLaunchKernelGGL(conv_tail_update_kernel, dim3(rows, (C + 255) / 256), dim3(256), 0, s, h, tail, row_start, slots, C, K);
     MIE_CHECK_LAUNCH("residual_conv (tail)");
   }
+  return 0;
+}
+
+// x points at the first of C columns (rows ldx floats apart); taps [C, K], bias [C] or null; tail [slots, max(1, K - 1), C];
+// u [tokens, C].  move_tail: every row of the step is one token, and the tail moves on here.
+MIE_EXPORT int mie_short_conv(const float* x, long ldx, const float* taps, const float* bias, float* tail, const int* token_row,
+                              const int* row_start, const int* slots, float* u, int tokens, int C, int K, int act, int move_tail,
+                              hipStream_t s) {
+  if (tokens <= 0) return 0;
+  if (C <= 0 || K < 1 || K > 64 || ldx < C) MIE_FAIL("short_conv: %d channels, %d taps (1 to 64), row stride %ld", C, K, ldx);
+  if (act < MIE_ACT_NONE || act > MIE_ACT_RELU2) MIE_FAIL("short_conv: activation code %d", act);
+  if (!x || !taps || !tail || !token_row || !row_start || !slots || !u) MIE_FAIL("short_conv: operands");
+  int by = (C + 255) / 256;
+  by = by > 64 ? 64 : by;
+#define SC(K_)                                                                                                              \
+  hipLaunchKernelGGL(short_conv_kernel<K_>, dim3(tokens, by), dim3(256), 0, s, x, ldx, taps, bias, tail, token_row, row_start, \
+                     slots, u, C, K, act, move_tail)
+  switch (K) {
+    case 2: SC(2); break;
+    case 3: SC(3); break;
+    case 4: SC(4); break;
+    default: SC(0);
+  }
+#undef SC
+  MIE_CHECK_LAUNCH("short_conv");
+  return 0;
+}
+
+MIE_EXPORT int mie_conv_tail_move(const float* x, long ldx, float* tail, const int* row_start, const int* slots, int rows, int C,
+                                  int K, hipStream_t s) {
+  if (rows <= 0 || K <= 1) return 0;
+  if (C <= 0 || ldx < C || !x || !tail || !row_start || !slots) MIE_FAIL("conv_tail_move: %d channels, row stride %ld", C, ldx);
+  hipLaunchKernelGGL(conv_tail_move_kernel, dim3(rows, (C + 255) / 256), dim3(256), 0, s, x, ldx, tail, row_start, slots, C, K);
+  MIE_CHECK_LAUNCH("conv_tail_move");
   return 0;
 }

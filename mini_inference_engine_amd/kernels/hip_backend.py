@@ -410,6 +410,41 @@ class HipBackend(KernelBackend):
                                            intermediate, self.ACT_CODES[activation], self._stream()))
         return out
 
+    def linear_clamped_glu(self, x, w_gate_up, intermediate, limit, alpha, shift):
+        I = intermediate
+        if w_gate_up.shape[0] != 2 * I or x.shape[1] != w_gate_up.shape[1]:
+            raise ValueError(f"linear_clamped_glu: x {tuple(x.shape)}, w {tuple(w_gate_up.shape)}, intermediate {I}")
+        if not limit > 0:
+            raise ValueError(f"linear_clamped_glu: limit {limit} must be positive")
+        self._on_device(w_gate_up)
+        _rows_ok(w_gate_up, "linear_clamped_glu: w")
+        prepared = self._prepared(x, w_gate_up, None)
+        rows = eps = None
+        if prepared is not None:
+            rows, eps, xt = x.rows, x.eps, prepared["x"]
+        else:
+            xt = x.materialize() if isinstance(x, Normed) else x
+        if prepared is not None or self._skinny_ok(xt, w_gate_up, None):      # few rows: the gate in the product's epilogue
+            M = xt.shape[0] if rows is None else rows.shape[0]
+            out = torch.empty((M, I), dtype=torch.bfloat16, device=w_gate_up.device)
+            lib = self.lib("gemm_bf16")
+            library.check(lib, lib.mie_skinny_clamped_glu(
+                _ptr(xt), xt.stride(0), _ptr(w_gate_up), w_gate_up.stride(0), _ptr(out), out.stride(0), M, I, w_gate_up.shape[1],
+                float(limit), float(alpha), float(shift), _ptr(prepared["ss"]) if prepared else None,
+                prepared["tiles"] if prepared else 0, float(eps or 0.0), _ptr(rows), self._stream()))
+            return out
+        packed = self.act_dtype == torch.bfloat16 and w_gate_up.dtype == torch.bfloat16 and I % 8 == 0
+        gu = self.linear(xt, w_gate_up, out_dtype=torch.bfloat16 if packed else torch.float32)
+        out = torch.empty((gu.shape[0], I), dtype=self.act_dtype, device=gu.device)
+        lib = self.lib("gemm")
+        if packed:
+            library.check(lib, lib.mie_clamped_glu_bf16(_ptr(gu), gu.stride(0), _ptr(out), out.stride(0), gu.shape[0], I, float(limit),
+                                                        float(alpha), float(shift), self._stream()))
+        else:
+            library.check(lib, lib.mie_clamped_glu(_ptr(gu), gu.stride(0), _ptr(out), out.stride(0), _code(out.dtype), gu.shape[0], I,
+                                                   float(limit), float(alpha), float(shift), 0, self._stream()))
+        return out
+
     def linear_act(self, x, w, activation="relu2"):
         if activation not in self.ACT_CODES:
             raise ValueError(f"linear_act: activation {activation!r}")
@@ -893,7 +928,8 @@ class HipBackend(KernelBackend):
 
     def qkv_finish(self, sums, q_col, k_col, v_col, num_q_heads, num_kv_heads, dim, vdim, padded_dim, positions, inv_freq,
                    layout, k_cache, v_cache, slot_mapping, q_norm=None, k_norm=None, eps=0.0, q_head_scale=None,
-                   norm_per_head=False, col_bias=None, position_temperature=None):
+                   norm_per_head=False, col_bias=None, position_temperature=None, rotation_scale=1.0, conv=None,
+                   values_out=None, value_mix=None):
         self._on_device(sums, positions, inv_freq, k_cache, v_cache, slot_mapping, q_norm, k_norm, q_head_scale, col_bias)
         coef, every = 0.0, 0
         if position_temperature is not None:
@@ -931,12 +967,168 @@ class HipBackend(KernelBackend):
         # rows 64 bytes apart from a multiple of their length, as the attention kernels like their q rows
         q = torch.empty((T, Hq * P), dtype=self.act_dtype, device=sums.device)
         lib = self.lib("attention_prep")
+        if conv is not None or rotation_scale != 1.0 or values_out is not None or value_mix is not None:
+            return self._qkv_conv_finish(q, sums, q_col, k_col, v_col, Hq, Hkv, dim, vdim, P, page, positions, inv_freq, nf, layout,
+                                         k_cache, v_cache, slot_mapping, q_norm, k_norm, eps, rotation_scale, conv, values_out, value_mix,
+                                         plain=q_head_scale is None and col_bias is None and position_temperature is None
+                                         and (norm_per_head or (q_norm is None and k_norm is None)))
         library.check(lib, lib.mie_qkv_finish(
             _ptr(sums), sums.stride(0), q_col, k_col, -1 if v_col is None else v_col, _ptr(q_norm), _ptr(k_norm), float(eps),
             int(bool(norm_per_head)), _ptr(inv_freq), nf, self.LAYOUTS[layout], _ptr(q_head_scale), _ptr(positions), _ptr(slot_mapping), _ptr(q),
             _ptr(k_cache), _ptr(v_cache), _code(self.act_dtype), T, Hq, Hkv, dim, vdim, P, page, _ptr(col_bias), coef, every,
             self._stream()))
         return q
+
+    def _qkv_conv_finish(self, q, sums, q_col, k_col, v_col, Hq, Hkv, dim, vdim, P, page, positions, inv_freq, nf, layout, k_cache,
+                         v_cache, slot_mapping, q_norm, k_norm, eps, rotation_scale, conv, values_out, value_mix, plain):
+        """The part of ``qkv_finish`` that convolves the projections, scales the rotation or shares values (operands checked)
+        -> q."""
+        T, dev = sums.shape[0], sums.device
+        if not plain or layout != "half" or conv is None:
+            raise ValueError("qkv_finish: a scaled rotation and shared values are built for convolved projections whose halves turn, "
+                             "with norms head by head and without biases and temperatures")
+        taps, tail, step = conv
+        self._on_device(taps, tail, values_out)
+        C = (Hq + Hkv) * dim + Hkv * vdim
+        if k_col != q_col + Hq * dim or v_col != k_col + Hkv * dim:
+            raise ValueError("qkv_finish: convolved projections lie side by side")
+        if taps.dim() != 2 or taps.shape[0] != C:
+            raise ValueError(f"qkv_finish: taps {tuple(taps.shape)} for {C} channels")
+        K = taps.shape[1]
+        self._f32_vector(taps, C * K, "qkv_finish: taps")
+        self._check_tail("qkv_finish", tail, C, K, step, T)
+        other, mix = None, 0.0
+        if value_mix is not None:
+            mix, other = float(value_mix[0]), value_mix[1]
+            self._on_device(other)
+        for name, t in (("values_out", values_out), ("the values to mix with", other)):
+            if t is not None:
+                self._f32_vector(t, T * Hkv * vdim, f"qkv_finish: {name}")
+        single = step.num_rows == T
+        lib = self.lib("attention_prep")
+        library.check(lib, lib.mie_qkv_conv_finish(
+            _ptr(sums), sums.stride(0), q_col, _ptr(taps), _ptr(tail), _ptr(step.token_row), _ptr(step.row_start), _ptr(step.state_slots),
+            K, int(single), _ptr(q_norm), _ptr(k_norm), float(eps), _ptr(inv_freq), nf, float(rotation_scale), _ptr(positions),
+            _ptr(slot_mapping), _ptr(values_out), _ptr(other), mix, _ptr(q), _ptr(k_cache), _ptr(v_cache), _code(self.act_dtype), T, Hq,
+            Hkv, dim, vdim, P, page, self._stream()))
+        if not single:
+            self._move_tail(sums, q_col, C, K, tail, step)
+        return q
+
+    def _check_tail(self, what, tail, C, K, step, T):
+        if tail.dtype != torch.float32 or tuple(tail.shape[1:]) != (max(1, K - 1), C) or not tail.is_contiguous():
+            raise ValueError(f"{what}: tail {tuple(tail.shape)} for {K} taps of {C} channels")
+        self._check_rows(what, step, T)
+        if int(step.host["state_slots"].max()) >= tail.shape[0]:
+            raise ValueError(f"{what}: a state slot beyond the tail's slots")
+
+    def _move_tail(self, x, col, C, K, tail, step):
+        """The rows' last K - 1 inputs (columns [col, col + C) of x, operands checked) into their slots of ``tail``."""
+        lib = self.lib("recurrence")
+        library.check(lib, lib.mie_conv_tail_move(c_void_p(x.data_ptr() + 4 * col), x.stride(0), _ptr(tail), _ptr(step.row_start),
+                                                  _ptr(step.state_slots), step.num_rows, C, K, self._stream()))
+
+    def gate_heads(self, o, gate, gate_col, num_heads, vdim, padded_dim, out=None, scale=1.0):
+        self._on_device(o, gate, out)
+        H, P, T = num_heads, padded_dim, o.shape[0]
+        if tuple(o.shape) != (T, H * P) or not o.is_contiguous() or P < vdim:
+            raise ValueError(f"gate_heads: o {tuple(o.shape)} for {H} heads of {vdim} in {P}")
+        gp = self._f32_columns(gate, gate_col, H * vdim, "gate_heads: gate")
+        if gate.shape[0] != T:
+            raise ValueError("gate_heads: one gate row a token")
+        out = self._branch_out("gate_heads", out, T, H * vdim, o.device, o.dtype)
+        lib = self.lib("attention_prep")
+        library.check(lib, lib.mie_gate_heads(_ptr(o), _code(o.dtype), gp, gate.stride(0), _ptr(out), out.stride(0), T, H, vdim, P,
+                                              float(scale), self._stream()))
+        return out
+
+    def _branch_out(self, what, out, T, n, device, dtype=None):
+        dtype = dtype or self.act_dtype
+        if out is None:
+            return torch.empty((T, n), dtype=dtype, device=device)
+        if tuple(out.shape) != (T, n) or out.dtype != dtype or out.stride(1) != 1:
+            raise ValueError(f"{what}: out {tuple(out.shape)} {out.dtype}, expected {(T, n)} {dtype} with unit inner stride")
+        return out
+
+    # ---- recurrences with one decay a head and token
+    def short_conv(self, x, col, channels, taps, bias, tail, step, activation="none"):
+        self._on_device(x, taps, bias, tail)
+        C, T = channels, x.shape[0]
+        xp = self._f32_columns(x, col, C, "short_conv")
+        if taps.dim() != 2 or taps.shape[0] != C:
+            raise ValueError(f"short_conv: taps {tuple(taps.shape)} for {C} channels")
+        K = taps.shape[1]
+        self._f32_vector(taps, C * K, "short_conv: taps")
+        if bias is not None:
+            self._f32_vector(bias, C, "short_conv: bias")
+        if activation not in self.ACT_CODES:
+            raise ValueError(f"short_conv: activation {activation!r}")
+        self._check_tail("short_conv", tail, C, K, step, T)
+        u = torch.empty((T, C), dtype=torch.float32, device=x.device)
+        single = step.num_rows == T
+        lib = self.lib("recurrence")
+        library.check(lib, lib.mie_short_conv(xp, x.stride(0), _ptr(taps), _ptr(bias), _ptr(tail), _ptr(step.token_row),
+                                              _ptr(step.row_start), _ptr(step.state_slots), _ptr(u), T, C, K,
+                                              self.ACT_CODES[activation], int(single), self._stream()))
+        if not single:
+            self._move_tail(x, col, C, K, tail, step)
+        return u
+
+    def _check_state(self, what, state, shape, step, T):
+        if state.dtype != torch.float32 or tuple(state.shape[1:]) != tuple(shape) or not state.is_contiguous():
+            raise ValueError(f"{what}: state {tuple(state.shape)}, expected [slots, {shape}]")
+        self._check_rows(what, step, T)
+        if int(step.host["state_slots"].max()) >= state.shape[0]:
+            raise ValueError(f"{what}: a state slot beyond the state's slots")
+
+    def state_space(self, u, b_col, c_col, sums, z_col, dt_col, num_heads, groups, state_dim, vdim, dt_bias, rate, skip,
+                    norm_groups, norm_weight, eps, state, step, out=None, scale=1.0):
+        self._on_device(u, sums, dt_bias, rate, skip, norm_weight, state, out)
+        H, N, dv, T = num_heads, state_dim, vdim, u.shape[0]
+        inner = H * dv
+        if sums.shape[0] != T or groups < 1 or H % groups or inner % norm_groups:
+            raise ValueError(f"state_space: {H} heads in {groups} groups, {inner} numbers in {norm_groups} parts, {sums.shape[0]} and {T} tokens")
+        self._f32_columns(u, 0, inner, "state_space: x")
+        self._f32_columns(u, b_col, groups * N, "state_space: B")
+        self._f32_columns(u, c_col, groups * N, "state_space: C")
+        zp = self._f32_columns(sums, z_col, inner, "state_space: z")
+        dtp = self._f32_columns(sums, dt_col, H, "state_space: dt")
+        for name, t, n in (("dt_bias", dt_bias, H), ("rate", rate, H), ("skip", skip, H), ("norm_weight", norm_weight, inner)):
+            self._f32_vector(t, n, f"state_space: {name}")
+        self._check_state("state_space", state, (H, N, dv), step, T)
+        out = self._branch_out("state_space", out, T, inner, u.device)
+        gates = torch.empty((2, T, H), dtype=torch.float32, device=u.device)
+        o = torch.empty((T, inner), dtype=torch.float32, device=u.device)
+        lib = self.lib("matrix_state")
+        library.check(lib, lib.mie_state_space(
+            _ptr(u), u.stride(0), b_col, c_col, zp, dtp, sums.stride(0), _ptr(dt_bias), _ptr(rate), _ptr(skip), _ptr(norm_weight),
+            float(eps), float(scale), _ptr(state), _ptr(step.row_start), _ptr(step.state_slots), _ptr(gates[0]), _ptr(gates[1]), _ptr(o),
+            _ptr(out), _code(out.dtype), out.stride(0), T, step.num_rows, H, groups, N, dv, norm_groups, self._stream()))
+        return out
+
+    def mlstm(self, sums, cols, num_heads, dim, vdim, i_bias, f_bias, cap, q_scale, norm_weight, eps, state, normaliser, maximum,
+              step, out=None, scale=1.0):
+        self._on_device(sums, i_bias, f_bias, norm_weight, state, normaliser, maximum, out)
+        H, d, dv, T = num_heads, dim, vdim, sums.shape[0]
+        for name, n in (("q", H * d), ("k", H * d), ("v", H * dv), ("g", H * dv), ("i", H), ("f", H)):
+            self._f32_columns(sums, cols[name], n, f"mlstm: {name}")
+        for name, t, n in (("i_bias", i_bias, H), ("f_bias", f_bias, H), ("norm_weight", norm_weight, H * dv)):
+            self._f32_vector(t, n, f"mlstm: {name}")
+        if not cap > 0:
+            raise ValueError(f"mlstm: cap {cap}")
+        self._check_state("mlstm", state, (H, d, dv), step, T)
+        self._f32_vector(normaliser, state.shape[0] * H * d, "mlstm: normaliser")
+        self._f32_vector(maximum, state.shape[0] * H, "mlstm: maximum")
+        out = self._branch_out("mlstm", out, T, H * dv, sums.device)
+        gates = torch.empty((4, T, H), dtype=torch.float32, device=sums.device)
+        o = torch.empty((T, H * dv), dtype=torch.float32, device=sums.device)
+        lib = self.lib("matrix_state")
+        library.check(lib, lib.mie_mlstm(
+            _ptr(sums), sums.stride(0), cols["q"], cols["k"], cols["v"], cols["g"], cols["i"], cols["f"], _ptr(i_bias), _ptr(f_bias),
+            float(cap), float(q_scale), _ptr(norm_weight), float(eps), float(scale), _ptr(state), _ptr(normaliser), _ptr(maximum),
+            _ptr(step.row_start), _ptr(step.state_slots), _ptr(gates[0]), _ptr(gates[1]), _ptr(gates[2]), _ptr(gates[3]), _ptr(o),
+            _ptr(out), _code(out.dtype), out.stride(0), T, step.num_rows, H, d, dv, self._stream()))
+        return out
 
     def head_gate_(self, o, gate, gate_col, num_heads, head_dim):
         self._on_device(o, gate)
@@ -1233,9 +1425,16 @@ class HipBackend(KernelBackend):
             Hq, Hkv, D, pending.page, float(scale), int(window or 0), partition, self._stream()))
         return out
 
+    def _in_log2(self, table):
+        """A table the matrix-core kernels add to scores or sinks, in their units of log2 e; made once a table."""
+        held = self._log2_tables.get(table.data_ptr())
+        if held is None or held[0] is not table:
+            held = self._log2_tables[table.data_ptr()] = (table, (table * 1.4426950408889634).contiguous())
+        return held[1]
+
     def paged_attention(self, qkv, num_q_heads, num_kv_heads, head_dim, k_cache, v_cache, group, step, scale,
                         window, sink=None, weights="softmax", softcap=None, chunk=None, head_bias=None,
-                        distance_bias=None, force_generic: bool = False, num_splits: int | None = None):
+                        distance_bias=None, keep_first: int = 0, force_generic: bool = False, num_splits: int | None = None):
         Hq, Hkv, D = num_q_heads, num_kv_heads, head_dim
         dist_n = 0
         if distance_bias is not None:
@@ -1244,7 +1443,16 @@ class HipBackend(KernelBackend):
                 raise ValueError(f"paged_attention: distance_bias {tuple(distance_bias.shape)} for {Hq} query heads")
             dist_n = distance_bias.shape[1]
             self._f32_vector(distance_bias, Hq * dist_n, "paged_attention: distance_bias")
+        head_sinks = None
+        if isinstance(sink, torch.Tensor):          # one a query head
+            self._on_device(sink)
+            self._f32_vector(sink, Hq, "paged_attention: sinks")
+            head_sinks, sink = sink, 0.0
         has_sink, sink = int(sink is not None), float(sink or 0.0)
+        keep_first = int(keep_first)
+        if keep_first < 0 or (keep_first and not window):
+            raise ValueError(f"paged_attention: {keep_first} kept first keys belong beside a window")
+        kept = bool(keep_first) or head_sinks is not None
         if weights not in ("softmax", "sigmoid"):
             raise ValueError(f"paged_attention: weights {weights!r} (softmax or sigmoid)")
         sigmoid = weights == "sigmoid"
@@ -1257,21 +1465,21 @@ class HipBackend(KernelBackend):
                 raise ValueError("paged_attention: a bias per head goes with sigmoid weights")
             self._on_device(head_bias)
             self._f32_vector(head_bias, Hq, "paged_attention: head_bias")
-        scored = sigmoid or softcap is not None or chunk is not None or distance_bias is not None
+        scored = sigmoid or softcap is not None or chunk is not None or distance_bias is not None or kept
         biased = distance_bias is not None and not sigmoid and softcap is None and chunk is None and not has_sink
-        if scored and not sigmoid and not biased:
+        only_kept = kept and not (sigmoid or softcap is not None or chunk is not None or distance_bias is not None)
+        if kept and not only_kept:
+            force_generic, biased = True, False     # kept keys or sinks a head beside another variation: the 32-bit kernel
+        if scored and not sigmoid and not biased and not only_kept:
             force_generic = True            # a capped or chunked softmax: the 32-bit kernel computes it
         table2 = None
         if biased and qkv.dtype == torch.bfloat16 and not force_generic and D <= 256:
             # the matrix-core kernels work in units of log2 e: the table in those units, made once a table
-            key = distance_bias.data_ptr()
-            held = self._log2_tables.get(key)
-            if held is None or held[0] is not distance_bias:
-                held = self._log2_tables[key] = (distance_bias, (distance_bias * 1.4426950408889634).contiguous())
-            table2 = held[1]
+            table2 = self._in_log2(distance_bias)
+        sinks2 = self._in_log2(head_sinks) if head_sinks is not None and qkv.dtype == torch.bfloat16 and not force_generic and D <= 256 else None
         if isinstance(qkv, ProjectionSums):
             out = self._decode_attention_from_sums(qkv, Hq, Hkv, D, k_cache, v_cache, group, step, scale, window,
-                                                   force_generic or num_splits is not None or bool(has_sink))
+                                                   force_generic or num_splits is not None or bool(has_sink) or kept)
             if out is not None:
                 return out
             qkv = qkv.finish()
@@ -1287,6 +1495,8 @@ class HipBackend(KernelBackend):
             block_keys = lib.mie_decode_block_keys()
             # a row sees at most a chunk's keys: the splits are planned as for a window of that many
             reach = min(window or chunk, chunk or window) if (window or chunk) else None
+            if keep_first:              # the kept keys' blocks come before the window's
+                reach = window + -(-keep_first // 32) * 32
             partition, splits = self.decode_splits(done, Hq, Hkv, step.max_context, reach, block_keys, D)
             if num_splits is not None:
                 bound = min(step.max_context, reach + 32) if reach else step.max_context
@@ -1302,6 +1512,8 @@ class HipBackend(KernelBackend):
             if sigmoid:
                 library.check(lib, lib.mie_decode_attention_sigmoid(*args, int(chunk or 0), float(softcap or 0.0),
                                                                     _ptr(head_bias), self._stream()))
+            elif kept:
+                library.check(lib, lib.mie_decode_attention_kept(*args, keep_first, _ptr(sinks2), self._stream()))
             elif table2 is not None:
                 library.check(lib, lib.mie_decode_attention_biased(*args, _ptr(table2), dist_n, self._stream()))
             elif has_sink:
@@ -1323,6 +1535,8 @@ class HipBackend(KernelBackend):
             if sigmoid:
                 library.check(lib, lib.mie_prefill_attention_sigmoid(*args, int(chunk or 0), float(softcap or 0.0),
                                                                      _ptr(head_bias), self._stream()))
+            elif kept:
+                library.check(lib, lib.mie_prefill_attention_kept(*args, keep_first, _ptr(sinks2), self._stream()))
             elif table2 is not None:
                 library.check(lib, lib.mie_prefill_attention_biased(*args, _ptr(table2), dist_n, self._stream()))
             elif has_sink:
@@ -1339,7 +1553,8 @@ class HipBackend(KernelBackend):
                     end - done, Hq, Hkv, D, page, float(scale), int(window or 0), has_sink, sink)
             if scored:
                 library.check(lib, lib.mie_paged_attention_scored(*args, int(chunk or 0), float(softcap or 0.0), int(sigmoid),
-                                                                  _ptr(head_bias), _ptr(distance_bias), dist_n, self._stream()))
+                                                                  _ptr(head_bias), _ptr(distance_bias), dist_n, keep_first, _ptr(head_sinks),
+                                                                  self._stream()))
             else:
                 library.check(lib, lib.mie_paged_attention(*args, self._stream()))
         return out

@@ -34,6 +34,7 @@ register_kernel_module("gemm", {
     "mie_act_mul": [P, L, P, L, I, I, I, I, P],
     "mie_act_store": [P, L, P, L, I, I, I, I, P],
     "mie_clamped_glu": [P, L, P, L, I, I, I, F, F, F, I, P],
+    "mie_clamped_glu_bf16": [P, L, P, L, I, I, F, F, F, P],
 })
 register_kernel_module("grouped_gemm", {
     "mie_grouped_linear": [P, I, L, L, I, P, I, L, L, P, I, L, L, P, P, L, P, P, I, I, I, I, I, I, P, P],
@@ -53,10 +54,14 @@ register_kernel_module("recurrence", {
     "mie_rglru_scan": [P, P, P, P, L, P, P, L, P, P, P, P, P, P, I, I, I, I, F, P],
     "mie_rglru_scan_chunked": [P, P, P, P, L, P, P, L, P, P, P, P, P, P, I, I, I, I, F, I, I, P, P, P, P],
     "mie_residual_conv": [P, P, P, P, P, P, P, I, I, I, I, I, P],
+    "mie_short_conv": [P, L, P, P, P, P, P, P, P, I, I, I, I, I, P],
+    "mie_conv_tail_move": [P, L, P, P, P, I, I, I, P],
 })
 register_kernel_module("attention_prep", {
     "mie_qkv_finish": [P, L, I, I, I, P, P, F, I, P, I, I, P, P, P, P, P, P, I, I, I, I, I, I, I, I, P, F, I, P],
     "mie_head_gate": [P, I, P, L, I, I, I, P],
+    "mie_qkv_conv_finish": [P, L, I, P, P, P, P, P, I, I, P, P, F, P, I, F, P, P, P, P, F, P, P, P, I, I, I, I, I, I, I, I, P],
+    "mie_gate_heads": [P, I, P, L, P, L, I, I, I, I, F, P],
 })
 register_kernel_module("delta_rule", {
     "mie_delta_rule": [P, L, I, I, I, I, I, I, P, I, P, F, P, P, F, P, P, P, P, P, I, I, I, I, I, I, I, P, P, P],
@@ -64,9 +69,13 @@ register_kernel_module("delta_rule", {
 register_kernel_module("gla", {
     "mie_gla": [P, L, I, I, I, I, I, P, I, P, F, F, P, F, P, P, P, P, P, I, I, I, I, I, I, I, I, P, P, P, P],
 })
+register_kernel_module("matrix_state", {
+    "mie_state_space": [P, L, I, I, P, P, L, P, P, P, P, F, F, P, P, P, P, P, P, P, I, L, I, I, I, I, I, I, I, P],
+    "mie_mlstm": [P, L, I, I, I, I, I, I, P, P, F, F, P, F, F, P, P, P, P, P, P, P, P, P, P, P, I, L, I, I, I, I, I, P],
+})
 register_kernel_module("attention", {
     "mie_paged_attention": [P, L, P, P, P, I, P, I, P, P, I, I, I, I, I, F, I, I, F, P],
-    "mie_paged_attention_scored": [P, L, P, P, P, I, P, I, P, P, I, I, I, I, I, F, I, I, F, I, F, I, P, P, I, P],
+    "mie_paged_attention_scored": [P, L, P, P, P, I, P, I, P, P, I, I, I, I, I, F, I, I, F, I, F, I, P, P, I, I, P, P],
 })
 register_kernel_module("sampling", {
     "mie_sample": [P, L, P, P, P, P, I, I, P],
@@ -74,6 +83,7 @@ register_kernel_module("sampling", {
 register_kernel_module("gemm_bf16", {
     "mie_skinny_gemm": [P, L, P, L, P, L, I, I, I, I, P, I, P, L, P, P, I, F, P, P],
     "mie_skinny_qkv_rope": [P, L, P, L, P, L, P, P, P, P, P, P, I, I, I, I, I, I, P, I, F, P],
+    "mie_skinny_clamped_glu": [P, L, P, L, P, L, I, I, I, F, F, F, P, I, F, P, P],
     "mie_skinny_max_rows": [],
 })
 register_kernel_module("gemm_mid_bf16", {
@@ -88,6 +98,7 @@ register_kernel_module("attention_bf16", {
     "mie_decode_attention_sink": [P, L, P, P, P, P, P, P, I, P, I, I, I, I, I, F, I, I, I, F, P],
     "mie_decode_attention_sigmoid": [P, L, P, P, P, P, P, P, I, P, I, I, I, I, I, F, I, I, I, I, F, P, P],
     "mie_decode_attention_biased": [P, L, P, P, P, P, P, P, I, P, I, I, I, I, I, F, I, I, I, P, I, P],
+    "mie_decode_attention_kept": [P, L, P, P, P, P, P, P, I, P, I, I, I, I, I, F, I, I, I, I, P, P],
     "mie_decode_attention_from_sums": [P, I, L, L, P, P, P, P, P, P, P, I, P, I, I, I, I, I, F, I, I, P],
     "mie_decode_attention_static": [P, L, P, P, P, P, I, P, I, I, I, I, I, F, I, I, I, P],
     "mie_decode_attention_static_setup": [],
@@ -102,6 +113,7 @@ register_kernel_module("prefill_attention_bf16", {
     "mie_prefill_attention_sink": [P, L, P, P, P, P, I, P, P, I, I, I, I, I, I, I, F, I, F, P],
     "mie_prefill_attention_sigmoid": [P, L, P, P, P, P, I, P, P, I, I, I, I, I, I, I, F, I, I, F, P, P],
     "mie_prefill_attention_biased": [P, L, P, P, P, P, I, P, P, I, I, I, I, I, I, I, F, I, P, I, P],
+    "mie_prefill_attention_kept": [P, L, P, P, P, P, I, P, P, I, I, I, I, I, I, I, F, I, I, P, P],
 }, variants=_head_variants, flags=["-mllvm", "-amdgpu-mfma-vgpr-form"])
 # lt_gemm: host code only, the engine's own way into the library's matrix products (hipBLASLt) with the choice of
 # kernel per shape kept here.

@@ -225,7 +225,7 @@ class SoftmaxAttention(Mixer):
                            cache.k, cache.v, group.slot_mapping, q_norm=self.q_norm if self.qk_norm else None,
                            k_norm=self.k_norm if self.qk_norm else None, eps=self.eps,
                            q_head_scale=self.temperature if self.head_temperature else None,
-                           **self._finish_options())
+                           **opts)
         more = {}
         if self.distance_table is not None:
             more["distance_bias"] = self.distance_table

@@ -204,7 +204,8 @@ def ref_rotary_kv_store(qkv, positions, cos, sin, rotary_dim, Hq, Hkv, D, k_cach
 
 
 def ref_paged_attention(qkv, Hq, Hkv, D, k_cache, v_cache, block_tables, token_row, positions, scale, window,
-                        out_dtype, sink=None, weights="softmax", softcap=None, chunk=None, head_bias=None, distance_bias=None):
+                        out_dtype, sink=None, weights="softmax", softcap=None, chunk=None, head_bias=None, distance_bias=None,
+                        keep_first=0):
     """Token by token, keys gathered through the block table."""
     T = qkv.shape[0]
     P = k_cache.shape[2]
@@ -219,6 +220,8 @@ def ref_paged_attention(qkv, Hq, Hkv, D, k_cache, v_cache, block_tables, token_r
         if chunk is not None:
             lo = max(lo, p // chunk * chunk)
         keys = torch.arange(lo, p + 1, device=qkv.device)
+        if keep_first and lo > 0:
+            keys = torch.cat([torch.arange(0, min(keep_first, lo), device=qkv.device), keys])
         pages = bt[rows[t], keys // P]
         k = k_cache[pages, :, keys % P, :].double()          # [n, Hkv, D]
         v = v_cache[pages, :, :, keys % P].double()             # [n, Hkv, D]
@@ -234,9 +237,11 @@ def ref_paged_attention(qkv, Hq, Hkv, D, k_cache, v_cache, block_tables, token_r
         elif sink is None:
             pr = torch.softmax(s, dim=-1)
         else:               # one more term in the denominator, with no value
-            top = s.max(-1, keepdim=True).values.clamp(min=sink)
+            sk = sink.double().view(Hkv, g, 1) if isinstance(sink, torch.Tensor) else torch.tensor(float(sink), dtype=torch.float64,
+                                                                                                  device=qkv.device)
+            top = torch.maximum(s.max(-1, keepdim=True).values, sk)
             e = torch.exp(s - top)
-            pr = e / (e.sum(-1, keepdim=True) + torch.exp(sink - top))
+            pr = e / (e.sum(-1, keepdim=True) + torch.exp(sk - top))
         out[t] = torch.einsum("hgn,nhd->hgd", pr, v).reshape(Hq * D).to(out_dtype)
     return out
 
@@ -272,8 +277,14 @@ def ref_turn(x, positions, inv_freq, layout):
 
 
 def ref_qkv_finish(sums, q_col, k_col, v_col, Hq, Hkv, dim, vdim, P, positions, inv_freq, layout, k_cache, v_cache, slots,
-                   q_norm, k_norm, eps, q_head_scale, out_dtype, norm_per_head=False, col_bias=None, position_temperature=None):
+                   q_norm, k_norm, eps, q_head_scale, out_dtype, norm_per_head=False, col_bias=None, position_temperature=None,
+                   rotation_scale=1.0, conv=None, values_out=None, value_mix=None):
     T = sums.shape[0]
+    if conv is not None:
+        taps, tail, row_start, state_slots = conv
+        C = taps.shape[0]
+        sums = sums.double()
+        sums[:, q_col:q_col + C] = ref_short_conv(sums, q_col, C, taps, None, tail, row_start, state_slots)
     if col_bias is not None:
         sums = (sums.double() + col_bias.double()).float()
     q = sums[:, q_col:q_col + Hq * dim].double()
@@ -288,7 +299,15 @@ def ref_qkv_finish(sums, q_col, k_col, v_col, Hq, Hkv, dim, vdim, P, positions, 
         k = k * torch.rsqrt(k.pow(2).mean(-1, keepdim=True) + eps) * k_norm.double()
     q, k = q.reshape(T, Hq, dim), k.reshape(T, Hkv, dim)
     if inv_freq is not None:
+        n = 2 * inv_freq.numel()
         q, k = ref_turn(q, positions, inv_freq, layout), ref_turn(k, positions, inv_freq, layout)
+        q[..., :n] *= rotation_scale
+        k[..., :n] *= rotation_scale
+    if values_out is not None:
+        values_out.copy_(v.reshape(T, -1).float())
+    if value_mix is not None:
+        lam, other = value_mix
+        v = (1.0 - lam) * v + lam * other.double().view(v.shape)
     if q_head_scale is not None:
         q = q * q_head_scale.double()[None, :, None]
     if position_temperature is not None:
@@ -391,6 +410,75 @@ def ref_gla(sums, cols, H, d, dv, w_decay, decay_bias, tau, q_scale, norm_weight
         state[int(slots[row])] = S.float()
     out = out * torch.rsqrt(out.pow(2).mean(-1, keepdim=True) + eps) * norm_weight.double()
     return (out.view(T, H * dv) * g * torch.sigmoid(g)).to(out_dtype)
+
+
+def ref_short_conv(x, col, C, taps, bias, tail, row_start, slots, activation="none"):
+    K = taps.shape[1]
+    out = torch.empty(x.shape[0], C, dtype=torch.float64, device=x.device)
+    for r in range(len(slots)):
+        a, b, slot = int(row_start[r]), int(row_start[r + 1]), int(slots[r])
+        inp = torch.cat([tail[slot][:K - 1].double(), x[a:b, col:col + C].double()])
+        acc = torch.zeros(b - a, C, dtype=torch.float64, device=x.device) if bias is None else bias.double().expand(b - a, C).clone()
+        for j in range(K):
+            acc += inp[j:j + b - a] * taps[:, j].double()
+        out[a:b] = acc if activation == "none" else ref_act(acc, activation)
+        if K > 1:
+            tail[slot][:K - 1] = inp[-(K - 1):].float()
+    return out
+
+
+def ref_gate_heads(o, gate, gate_col, H, dv, P, scale, out_dtype):
+    T = o.shape[0]
+    g = torch.sigmoid(gate[:, gate_col:gate_col + H * dv].double())
+    return (scale * o.double().view(T, H, P)[..., :dv].reshape(T, H * dv) * g).to(out_dtype)
+
+
+def ref_state_space(u, b_col, c_col, sums, z_col, dt_col, H, G, N, dv, dt_bias, rate, skip, norm_groups, norm_weight, eps, state,
+                    row_start, slots, scale, out_dtype):
+    T, inner = u.shape[0], H * dv
+    x = u[:, :inner].double().view(T, H, dv)
+    B = u[:, b_col:b_col + G * N].double().view(T, G, N).repeat_interleave(H // G, 1)
+    C = u[:, c_col:c_col + G * N].double().view(T, G, N).repeat_interleave(H // G, 1)
+    dt = torch.nn.functional.softplus(sums[:, dt_col:dt_col + H].double() + dt_bias.double(), threshold=50)
+    keep = torch.exp(-rate.double() * dt)
+    y = torch.empty(T, H, dv, dtype=torch.float64, device=u.device)
+    for row in range(len(slots)):
+        S = state[int(slots[row])].double()
+        for t in range(int(row_start[row]), int(row_start[row + 1])):
+            S = keep[t][:, None, None] * S + (dt[t][:, None] * B[t])[:, :, None] * x[t][:, None, :]
+            y[t] = torch.einsum("hij,hi->hj", S, C[t]) + skip.double()[:, None] * x[t]
+        state[int(slots[row])] = S.float()
+    z = sums[:, z_col:z_col + inner].double()
+    y = (y.view(T, inner) * z * torch.sigmoid(z)).view(T, norm_groups, -1)
+    y = (y * torch.rsqrt(y.pow(2).mean(-1, keepdim=True) + eps)).view(T, inner)
+    return (scale * y * norm_weight.double()).to(out_dtype)
+
+
+def ref_mlstm(sums, cols, H, d, dv, i_bias, f_bias, cap, q_scale, norm_weight, eps, state, normaliser, maximum, row_start, slots,
+              scale, out_dtype):
+    T = sums.shape[0]
+    x = sums.double()
+    q = x[:, cols["q"]:cols["q"] + H * d].view(T, H, d) * q_scale
+    k = x[:, cols["k"]:cols["k"] + H * d].view(T, H, d)
+    v = x[:, cols["v"]:cols["v"] + H * dv].view(T, H, dv)
+    g = x[:, cols["g"]:cols["g"] + H * dv]
+    gi = cap * torch.tanh((x[:, cols["i"]:cols["i"] + H] + i_bias.double()) / cap)
+    gf = torch.nn.functional.logsigmoid(cap * torch.tanh((x[:, cols["f"]:cols["f"] + H] + f_bias.double()) / cap))
+    o = torch.empty(T, H, dv, dtype=torch.float64, device=sums.device)
+    for row in range(len(slots)):
+        slot = int(slots[row])
+        S, n, m = state[slot].double(), normaliser[slot].double(), maximum[slot].double()
+        for t in range(int(row_start[row]), int(row_start[row + 1])):
+            new = torch.maximum(gf[t] + m, gi[t])
+            keep, take = torch.exp(gf[t] + m - new), torch.exp(gi[t] - new)
+            S = keep[:, None, None] * S + take[:, None, None] * k[t][:, :, None] * v[t][:, None, :]
+            n = keep[:, None] * n + take[:, None] * k[t]
+            m = new
+            below = torch.maximum((n * q[t]).sum(-1).abs(), torch.exp(-m)) + 1e-6
+            o[t] = torch.einsum("hij,hi->hj", S, q[t]) / below[:, None]
+        state[slot], normaliser[slot], maximum[slot] = S.float(), n.float(), m.float()
+    o = (o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + eps)).view(T, H * dv)
+    return (scale * o * norm_weight.double() * torch.sigmoid(g)).to(out_dtype)
 
 
 def _fmix32(x):
@@ -548,12 +636,13 @@ class TorchBackend(KernelBackend):
                             k_cache, v_cache, slot_mapping)
 
     def paged_attention(self, qkv, num_q_heads, num_kv_heads, head_dim, k_cache, v_cache, group, step, scale,
-                        window, sink=None, weights="softmax", softcap=None, chunk=None, head_bias=None, distance_bias=None):
+                        window, sink=None, weights="softmax", softcap=None, chunk=None, head_bias=None, distance_bias=None,
+                        keep_first=0):
         self._count("paged_attention")
         return ref_paged_attention(qkv, num_q_heads, num_kv_heads, head_dim, k_cache, v_cache, group.block_tables,
                                    step.token_row, step.positions, scale, window, self.act_dtype, sink=sink,
                                    weights=weights, softcap=softcap, chunk=chunk, head_bias=head_bias,
-                                   distance_bias=distance_bias)
+                                   distance_bias=distance_bias, keep_first=keep_first)
 
     def residual_conv(self, h, taps, tail, step, out_dtype=None):
         self._count("residual_conv")
@@ -561,11 +650,43 @@ class TorchBackend(KernelBackend):
 
     def qkv_finish(self, sums, q_col, k_col, v_col, num_q_heads, num_kv_heads, dim, vdim, padded_dim, positions, inv_freq,
                    layout, k_cache, v_cache, slot_mapping, q_norm=None, k_norm=None, eps=0.0, q_head_scale=None,
-                   norm_per_head=False, col_bias=None, position_temperature=None):
+                   norm_per_head=False, col_bias=None, position_temperature=None, rotation_scale=1.0, conv=None,
+                   values_out=None, value_mix=None):
         self._count("qkv_finish")
+        if conv is not None:
+            conv = (conv[0], conv[1], conv[2].host["row_start"], conv[2].host["state_slots"])
         return ref_qkv_finish(sums, q_col, k_col, v_col, num_q_heads, num_kv_heads, dim, vdim, padded_dim, positions, inv_freq,
                               layout, k_cache, v_cache, slot_mapping, q_norm, k_norm, eps, q_head_scale, self.act_dtype,
-                              norm_per_head, col_bias, position_temperature)
+                              norm_per_head, col_bias, position_temperature, rotation_scale, conv, values_out, value_mix)
+
+    def linear_clamped_glu(self, x, w_gate_up, intermediate, limit, alpha, shift):
+        self._count("linear_clamped_glu")
+        if isinstance(x, Normed):
+            x = x.materialize()
+        gu = ref_linear(x, w_gate_up, None, torch.float32).double()
+        return ref_clamped_glu(gu, intermediate, limit, alpha, shift).to(self.act_dtype)
+
+    def gate_heads(self, o, gate, gate_col, num_heads, vdim, padded_dim, out=None, scale=1.0):
+        y = ref_gate_heads(o, gate, gate_col, num_heads, vdim, padded_dim, scale, self.act_dtype)
+        return y if out is None else out.copy_(y)
+
+    def short_conv(self, x, col, channels, taps, bias, tail, step, activation="none"):
+        self._count("short_conv")
+        return ref_short_conv(x, col, channels, taps, bias, tail, step.host["row_start"], step.host["state_slots"], activation).float()
+
+    def state_space(self, u, b_col, c_col, sums, z_col, dt_col, num_heads, groups, state_dim, vdim, dt_bias, rate, skip,
+                    norm_groups, norm_weight, eps, state, step, out=None, scale=1.0):
+        self._count("state_space")
+        y = ref_state_space(u, b_col, c_col, sums, z_col, dt_col, num_heads, groups, state_dim, vdim, dt_bias, rate, skip, norm_groups,
+                            norm_weight, eps, state, step.host["row_start"], step.host["state_slots"], scale, self.act_dtype)
+        return y if out is None else out.copy_(y)
+
+    def mlstm(self, sums, cols, num_heads, dim, vdim, i_bias, f_bias, cap, q_scale, norm_weight, eps, state, normaliser, maximum,
+              step, out=None, scale=1.0):
+        self._count("mlstm")
+        y = ref_mlstm(sums, cols, num_heads, dim, vdim, i_bias, f_bias, cap, q_scale, norm_weight, eps, state, normaliser, maximum,
+                      step.host["row_start"], step.host["state_slots"], scale, self.act_dtype)
+        return y if out is None else out.copy_(y)
 
     def head_gate_(self, o, gate, gate_col, num_heads, head_dim):
         o.copy_(ref_head_gate(o, gate, gate_col, num_heads, head_dim))
