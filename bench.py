@@ -3,7 +3,7 @@ Llama-2-7B or Llama-3-8B), random weights.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch 8] [--shape tinyllama] [--context N] [--layers L]
     python bench.py --kernels [--shape ...] [--batch 8] [--context N]     each dominant kernel alone
-    python bench.py --design zifelorn|vezodra|mutusun|labirax [--design-sizes 1024,2048] [--layers R] [--batch 8] [--context 1024]
+    python bench.py --design zifelorn|vezodra|mutusun|labirax|pokulorn [--design-sizes 1024,2048] [--layers R] [--batch 8] [--context 1024]
                                                  that design beside Llama at equal layer sizes (R runs of its layers)
 
 A step is one decode step of the engine (schedule, batch, captured forward, sampling,
@@ -471,10 +471,27 @@ LABIRAX_SIZES = {
 }
 
 
+# Pokulorn layer sizes of the same widths: a run of three layers is full attention beside the state space, attention under a
+# window with kept first tokens, and the matrix memory, each with the dense clamped feed-forward.
+POKULORN_SIZES = {
+    "1024": dict(vocab=32000, width=1024, ff=2816, heads=16, kv_heads=4, dim=64, window=1024, keep_first=4, pair_heads=8,
+                 pair_kv_heads=2, pair_dim=128, ssm_heads=16, ssm_vdim=64, ssm_state=128, ssm_groups=4, mem_heads=4, mem_dim=128,
+                 mem_vdim=256),
+    "2048": dict(vocab=32000, width=2048, ff=5632, heads=32, kv_heads=8, dim=64, window=1024, keep_first=4, pair_heads=16,
+                 pair_kv_heads=4, pair_dim=128, ssm_heads=32, ssm_vdim=64, ssm_state=128, ssm_groups=8, mem_heads=8, mem_dim=128,
+                 mem_vdim=256),
+}
+
+
 def design_configs(design: str, size: str, repeats: int):
     """(the design's configuration, Llama's of the same width, head count, feed-forward size, vocabulary and layer count)."""
-    from mini_inference_engine_amd.config import LabiraxConfig, LlamaConfig, MutusunConfig, VezodraConfig, ZifelornConfig
-    if design == "labirax":
+    from mini_inference_engine_amd.config import (LabiraxConfig, LlamaConfig, MutusunConfig, PokulornConfig, VezodraConfig,
+                                                  ZifelornConfig)
+    if design == "pokulorn":
+        from mini_inference_engine_amd.models.pokulorn import _shape
+        z = POKULORN_SIZES[size]
+        cfg, layers = PokulornConfig.from_dict(_shape(repeats=repeats, **z)), 3 * repeats
+    elif design == "labirax":
         from mini_inference_engine_amd.models.labirax import _shape
         z = LABIRAX_SIZES[size]
         cfg = LabiraxConfig.from_dict(_shape(repeats=repeats, shared=1, **{k: v for k, v in z.items() if k != "ff"}))
@@ -534,7 +551,7 @@ def measure_designs(args) -> int:
 
 def main() -> int:
     ap = argparse.ArgumentParser()
-    ap.add_argument("--design", choices=["zifelorn", "vezodra", "mutusun", "labirax"], default=None,
+    ap.add_argument("--design", choices=["zifelorn", "vezodra", "mutusun", "labirax", "pokulorn"], default=None,
                     help="instead of the default workload: that design beside Llama at equal layer sizes (decode and prefill)")
     ap.add_argument("--design-sizes", default=None, help="comma-separated widths of --design (default: all of 1024, 2048)")
     ap.add_argument("--gpus", type=int, default=1)

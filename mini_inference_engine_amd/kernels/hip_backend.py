@@ -1081,6 +1081,20 @@ class HipBackend(KernelBackend):
         if int(step.host["state_slots"].max()) >= state.shape[0]:
             raise ValueError(f"{what}: a state slot beyond the state's slots")
 
+    STATE_CHUNK = 64         # tokens a chunk of the matrix-state recurrences; rows up to this long run whole
+
+    def _state_chunks(self, step, H, d, dv, device, normaliser=False):
+        """(longest row, chunks a row or 0, scratch for the chunks' states, normalisers and decays).  Rows of many tokens run in
+        chunks side by side (whether a step takes this path depends on its longest row alone; the two paths differ by rounding,
+        so the 32-bit mode keeps to one)."""
+        longest = int(getattr(step, "max_row_tokens", 0) or (step.host["row_start"][1:] - step.host["row_start"][:-1]).max())
+        if longest <= self.STATE_CHUNK or self.true_fp32:
+            return longest, 0, None, None, None
+        chunks = -(-longest // self.STATE_CHUNK)
+        units = step.num_rows * chunks
+        make = lambda *shape: torch.empty((units, H, *shape), dtype=torch.float32, device=device)       # noqa: E731
+        return longest, chunks, make(d, dv), make(d) if normaliser else None, make()
+
     def state_space(self, u, b_col, c_col, sums, z_col, dt_col, num_heads, groups, state_dim, vdim, dt_bias, rate, skip,
                     norm_groups, norm_weight, eps, state, step, out=None, scale=1.0):
         self._on_device(u, sums, dt_bias, rate, skip, norm_weight, state, out)
@@ -1098,12 +1112,14 @@ class HipBackend(KernelBackend):
         self._check_state("state_space", state, (H, N, dv), step, T)
         out = self._branch_out("state_space", out, T, inner, u.device)
         gates = torch.empty((2, T, H), dtype=torch.float32, device=u.device)
+        _, chunks, starts, _, ends = self._state_chunks(step, H, N, dv, u.device)
         o = torch.empty((T, inner), dtype=torch.float32, device=u.device)
         lib = self.lib("matrix_state")
         library.check(lib, lib.mie_state_space(
             _ptr(u), u.stride(0), b_col, c_col, zp, dtp, sums.stride(0), _ptr(dt_bias), _ptr(rate), _ptr(skip), _ptr(norm_weight),
             float(eps), float(scale), _ptr(state), _ptr(step.row_start), _ptr(step.state_slots), _ptr(gates[0]), _ptr(gates[1]), _ptr(o),
-            _ptr(out), _code(out.dtype), out.stride(0), T, step.num_rows, H, groups, N, dv, norm_groups, self._stream()))
+            _ptr(out), _code(out.dtype), out.stride(0), T, step.num_rows, H, groups, N, dv, norm_groups,
+            chunks, _ptr(starts), _ptr(ends), self._stream()))
         return out
 
     def mlstm(self, sums, cols, num_heads, dim, vdim, i_bias, f_bias, cap, q_scale, norm_weight, eps, state, normaliser, maximum,
@@ -1121,13 +1137,15 @@ class HipBackend(KernelBackend):
         self._f32_vector(maximum, state.shape[0] * H, "mlstm: maximum")
         out = self._branch_out("mlstm", out, T, H * dv, sums.device)
         gates = torch.empty((4, T, H), dtype=torch.float32, device=sums.device)
+        longest, chunks, starts, n_starts, ends = self._state_chunks(step, H, d, dv, sums.device, normaliser=True)
         o = torch.empty((T, H * dv), dtype=torch.float32, device=sums.device)
         lib = self.lib("matrix_state")
         library.check(lib, lib.mie_mlstm(
             _ptr(sums), sums.stride(0), cols["q"], cols["k"], cols["v"], cols["g"], cols["i"], cols["f"], _ptr(i_bias), _ptr(f_bias),
             float(cap), float(q_scale), _ptr(norm_weight), float(eps), float(scale), _ptr(state), _ptr(normaliser), _ptr(maximum),
             _ptr(step.row_start), _ptr(step.state_slots), _ptr(gates[0]), _ptr(gates[1]), _ptr(gates[2]), _ptr(gates[3]), _ptr(o),
-            _ptr(out), _code(out.dtype), out.stride(0), T, step.num_rows, H, d, dv, self._stream()))
+            _ptr(out), _code(out.dtype), out.stride(0), T, step.num_rows, H, d, dv, longest, chunks, _ptr(starts), _ptr(n_starts), _ptr(ends),
+            self._stream()))
         return out
 
     def head_gate_(self, o, gate, gate_col, num_heads, head_dim):

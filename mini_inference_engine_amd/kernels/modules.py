@@ -70,8 +70,8 @@ register_kernel_module("gla", {
     "mie_gla": [P, L, I, I, I, I, I, P, I, P, F, F, P, F, P, P, P, P, P, I, I, I, I, I, I, I, I, P, P, P, P],
 })
 register_kernel_module("matrix_state", {
-    "mie_state_space": [P, L, I, I, P, P, L, P, P, P, P, F, F, P, P, P, P, P, P, P, I, L, I, I, I, I, I, I, I, P],
-    "mie_mlstm": [P, L, I, I, I, I, I, I, P, P, F, F, P, F, F, P, P, P, P, P, P, P, P, P, P, P, I, L, I, I, I, I, I, P],
+    "mie_state_space": [P, L, I, I, P, P, L, P, P, P, P, F, F, P, P, P, P, P, P, P, I, L, I, I, I, I, I, I, I, I, P, P, P],
+    "mie_mlstm": [P, L, I, I, I, I, I, I, P, P, F, F, P, F, F, P, P, P, P, P, P, P, P, P, P, P, I, L, I, I, I, I, I, I, I, P, P, P, P],
 })
 register_kernel_module("attention", {
     "mie_paged_attention": [P, L, P, P, P, I, P, I, P, P, I, I, I, I, I, F, I, I, F, P],
