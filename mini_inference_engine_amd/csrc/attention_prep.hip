@@ -216,6 +216,179 @@ qkv_conv_finish_kernel(ConvFinishArgs a) {
   }
 }
 
+// The same for steps with rows of many tokens: a workgroup a (16 tokens, share of the heads), a wave a head for all of the 16,
+// four at a time.  A lane owns E channels of the head and carries their last inputs along, so that every number is read
+// once; the angles' cosines and sines of the 16 tokens are made once a workgroup; where the 16 tokens fill a stretch of
+// 16 slots of a page, the values of four go out as one run a dim.
+template <typename TO, int KT, int E>
+__global__ void __launch_bounds__(256)
+qkv_conv_finish_tile_kernel(ConvFinishArgs a, int tokens) {
+  constexpr int TT = 16, U = 4, keep = KT - 1;
+  extern __shared__ __align__(16) float lds[];
+  const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, P = a.P;
+  float* cs = lds;                                            // [TT][nf] cosines, then sines
+  float* sn = cs + TT * a.nf;
+  float* mine = lds + 2 * TT * a.nf + (size_t)wv * U * P;     // the wave's normed heads of four tokens
+  const int t_first = blockIdx.x * TT, t_end = t_first + TT < tokens ? t_first + TT : tokens;
+  for (int i = threadIdx.x; i < TT * a.nf; i += 256) {
+    const int tt = i / a.nf, f = i - tt * a.nf;
+    float s, c;
+    sincosf((float)a.positions[t_first + tt < t_end ? t_first + tt : t_end - 1] * a.inv_freq[f], &s, &c);
+    cs[i] = c * a.rot_scale;
+    sn[i] = s * a.rot_scale;
+  }
+  __syncthreads();
+  // whether the 16 tokens fill one stretch of 16 slots of a page, in order (a row's tokens mostly do)
+  const int slot0 = a.slots[t_first];
+  const bool run = t_end - t_first == TT && a.page % TT == 0 && slot0 % TT == 0 &&
+                   __builtin_amdgcn_ballot_w64(a.slots[t_first + (lane & (TT - 1) & (t_end - t_first - 1))] !=
+                                               slot0 + (lane & (TT - 1) & (t_end - t_first - 1))) == 0;
+  const int jobs = a.Hq + 2 * a.Hkv;
+  for (int job = blockIdx.y * 4 + wv; job < jobs; job += gridDim.y * 4) {
+    const bool is_q = job < a.Hq, is_v = job >= a.Hq + a.Hkv;
+    const int h = is_q ? job : is_v ? job - a.Hq - a.Hkv : job - a.Hq;
+    const int n = is_v ? a.vdim : a.dim;
+    const int c0 = is_q ? h * a.dim : is_v ? (a.Hq + a.Hkv) * a.dim + h * a.vdim : (a.Hq + h) * a.dim;
+    const float* __restrict__ w = is_q ? a.q_norm : a.k_norm;
+    float tp[E][KT], win[E][keep], wn[E];
+    int ch[E];                                                // the lane's channels, clamped into the head
+#pragma unroll
+    for (int e = 0; e < E; ++e) {
+      const int d = lane + 64 * e;
+      ch[e] = c0 + (d < n ? d : n - 1);
+      wn[e] = !is_v && w && d < n ? w[d] : 1.f;
+#pragma unroll
+      for (int k = 0; k < KT; ++k) tp[e][k] = a.taps[(size_t)ch[e] * KT + k];
+    }
+#pragma unroll 1
+    for (int g = 0; g < TT; g += U) {
+      float x[U][E], y[U][E], ss[U];
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        const int t = t_first + g + u < t_end ? t_first + g + u : t_end - 1;
+#pragma unroll
+        for (int e = 0; e < E; ++e) x[u][e] = a.sums[(size_t)t * a.ld + a.col + ch[e]];
+      }
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        const int t = t_first + g + u < t_end ? t_first + g + u : t_end - 1;
+        const int r = a.token_row[t], j = t - a.row_start[r];
+        if (g + u == 0 || j == 0) {                           // the inputs before this token: of its row, or from the tail
+          const float* __restrict__ tl = a.tail + (size_t)a.state_slots[r] * keep * a.C;
+#pragma unroll
+          for (int e = 0; e < E; ++e)
+#pragma unroll
+            for (int i = 0; i < keep; ++i) {
+              const int back = keep - i;
+              win[e][i] = back <= j ? a.sums[(size_t)(t - back) * a.ld + a.col + ch[e]] : tl[(size_t)(keep + j - back) * a.C + ch[e]];
+            }
+        }
+        ss[u] = 0.f;
+#pragma unroll
+        for (int e = 0; e < E; ++e) {
+          float acc = 0.f;
+#pragma unroll
+          for (int i = 0; i < keep; ++i) acc = fmaf(tp[e][i], win[e][i], acc);
+          acc = fmaf(tp[e][keep], x[u][e], acc);
+#pragma unroll
+          for (int i = 0; i + 1 < keep; ++i) win[e][i] = win[e][i + 1];
+          win[e][keep - 1] = x[u][e];
+          y[u][e] = lane + 64 * e < n ? acc : 0.f;
+          ss[u] = fmaf(y[u][e], y[u][e], ss[u]);
+        }
+      }
+      if (is_v) {
+        struct alignas(U * sizeof(TO)) Four { TO v[U]; } vals[E];
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+          const int t = t_first + g + u;
+          if (t < t_end) {
+            const size_t at = ((size_t)t * a.Hkv + h) * a.vdim;
+#pragma unroll
+            for (int e = 0; e < E; ++e) {
+              const int d = lane + 64 * e;
+              float v = y[u][e];
+              if (d < n) {
+                if (a.values_out) a.values_out[at + d] = v;
+                if (a.mix_other) v = (1.0f - a.mix) * v + a.mix * a.mix_other[at + d];
+              }
+              vals[e].v[u] = from_float<TO>(v);
+              if (!run && d < P) {
+                const int slot = a.slots[t];
+                ((TO*)a.v_cache)[(((size_t)(slot / a.page) * a.Hkv + h) * P + d) * a.page + slot % a.page] = vals[e].v[u];
+              }
+            }
+          }
+        }
+        if (run) {
+#pragma unroll
+          for (int e = 0; e < E; ++e)
+            if (lane + 64 * e < P)
+              *reinterpret_cast<Four*>((TO*)a.v_cache + (((size_t)(slot0 / a.page) * a.Hkv + h) * P + lane + 64 * e) * a.page +
+                                       slot0 % a.page + g) = vals[e];
+        }
+        continue;
+      }
+      if (w) {
+#pragma unroll
+        for (int o = 32; o > 0; o >>= 1)
+#pragma unroll
+          for (int u = 0; u < U; ++u) ss[u] += __shfl_xor(ss[u], o, 64);
+      }
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        const float rms = w ? 1.0f / sqrtf(ss[u] / (float)n + a.eps) : 1.f;
+#pragma unroll
+        for (int e = 0; e < E; ++e) {
+          y[u][e] *= rms * wn[e];
+          if (lane + 64 * e < P) mine[u * P + lane + 64 * e] = y[u][e];
+        }
+      }
+      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+      __builtin_amdgcn_wave_barrier();
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        const int t = t_first + g + u;
+        if (t < t_end) {
+          const int slot = a.slots[t];
+          TO* __restrict__ dst = is_q ? (TO*)a.q_out + ((size_t)t * a.Hq + h) * P
+                                      : (TO*)a.k_cache + (((size_t)(slot / a.page) * a.Hkv + h) * a.page + slot % a.page) * P;
+#pragma unroll
+          for (int e = 0; e < E; ++e) {
+            const int d = lane + 64 * e;
+            if (d < P) {
+              float o = y[u][e];
+              if (d < 2 * a.nf) {
+                const bool low = d < a.nf;
+                const int f = low ? d : d - a.nf;
+                const float c = cs[(g + u) * a.nf + f], s = sn[(g + u) * a.nf + f], other = mine[u * P + (low ? d + a.nf : f)];
+                o = low ? fmaf(o, c, -(other * s)) : fmaf(o, c, other * s);
+              }
+              dst[d] = from_float<TO>(o);
+            }
+          }
+        }
+      }
+      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+      __builtin_amdgcn_wave_barrier();
+    }
+  }
+}
+
+template <typename TO, int KT>
+static void qkv_conv_tile_launch(const ConvFinishArgs& a, int tokens, hipStream_t s) {
+  const int e = (a.P + 63) / 64;
+  const size_t lds = ((size_t)2 * 16 * a.nf + (size_t)4 * 4 * a.P) * sizeof(float);
+  const int tiles = (tokens + 15) / 16;
+  int parts = (a.Hq + 2 * a.Hkv + 3) / 4;
+  while (parts > 1 && (long)tiles * parts > 1536) parts = (parts + 1) / 2;       // a few workgroups a compute unit
+#define QCT(E_) hipLaunchKernelGGL((qkv_conv_finish_tile_kernel<TO, KT, E_>), dim3(tiles, parts), dim3(256), lds, s, a, tokens)
+  if (e <= 1) QCT(1);
+  else if (e == 2) QCT(2);
+  else QCT(4);
+#undef QCT
+}
+
 MIE_EXPORT const char* attention_prep_last_error() { return g_mie_error; }
 
 MIE_EXPORT int mie_qkv_finish(const float* sums, long ld, int q_col, int k_col, int v_col, const float* q_norm,
@@ -283,6 +456,21 @@ MIE_EXPORT int mie_qkv_conv_finish(const float* sums, long ld, int col, const fl
   ConvFinishArgs a{sums, ld, col, taps, tail, token_row, row_start, state_slots, K, move_tail, q_norm, k_norm, eps, inv_freq, nf,
                    rot_scale, positions, slots, values_out, mix_other, mix, q_out, k_cache, v_cache, Hq, Hkv, dim, vdim, P, page, C,
                    row_floats};
+  // rows of many tokens: 16 tokens a workgroup (the angles' table of a workgroup has to fit beside the heads)
+  if (tokens >= 64 && !move_tail && K >= 2 && K <= 4 && P <= 256 && nf <= 128) {
+#define QCT_K(T_)                                        \
+  switch (K) {                                           \
+    case 2: qkv_conv_tile_launch<T_, 2>(a, tokens, s); break; \
+    case 3: qkv_conv_tile_launch<T_, 3>(a, tokens, s); break; \
+    default: qkv_conv_tile_launch<T_, 4>(a, tokens, s); \
+  }
+    if (dtype == MIE_F32) { QCT_K(float) }
+    else if (dtype == MIE_BF16) { QCT_K(bf16) }
+    else MIE_FAIL("qkv_conv_finish: dtype code %d", dtype);
+#undef QCT_K
+    MIE_CHECK_LAUNCH("qkv_conv_finish (tiles)");
+    return 0;
+  }
   const size_t lds = (size_t)4 * row_floats * sizeof(float);
   int parts = (Hq + 2 * Hkv + 3) / 4;
   const int most = tokens >= 1024 ? 4 : 16;

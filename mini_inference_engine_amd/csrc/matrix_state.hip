@@ -336,14 +336,14 @@ template <int NT>
 __global__ void __launch_bounds__(256)
 chunk_outputs_kernel(ChunkArgs p) {
   constexpr int VS = 16 * NT + 4, PS = CH + 4;
-  constexpr int QKS = 2 * CH * QS + DB * VS, FLOATS = QKS > CH * VS ? QKS : CH * VS;
-  __shared__ __align__(16) float buf[FLOATS];
-  __shared__ __align__(16) float sp[CH * PS];
+  constexpr int QKS = 2 * CH * QS + DB * VS, VP = CH * VS + CH * PS, FLOATS = QKS > VP ? QKS : VP;
+  __shared__ __align__(16) float buf[FLOATS];           // q, k, S_0; after the products over the state rows v and the weights
   __shared__ float A[CH], cc[CH], sn[DB], rows_sum[CH];
   float* sq = buf;
   float* sk = buf + CH * QS;
   float* ss = buf + 2 * CH * QS;
-  float* sv = buf;                              // after the products over the state rows
+  float* sv = buf;
+  float* sp = buf + CH * VS;
   const ScanArgs& a = p.s;
   CHUNK_OF_ROW;
   const int h = blockIdx.y, v0 = blockIdx.z * 16 * NT, tid = threadIdx.x;
@@ -421,6 +421,13 @@ chunk_outputs_kernel(ChunkArgs p) {
       }
     }
   }
+  f32x4 rv[NT];
+#pragma unroll
+  for (int i = 0; i < NT; ++i) {
+    const int e = tid + 256 * i, t = e / (4 * NT);
+    rv[i] = load4(vp + (size_t)(t < nt ? t : nt - 1) * a.ld_v, v0 + 4 * (e % (4 * NT)), a.dv, p.vec);     // beyond the end: meets zeros
+  }
+  __syncthreads();                              // everybody is done with q, k and S_0
   // a lane holds rows (tokens) 4 g + e of the wave's 16 and column n of every tile
   float At[4], eA[4], sum[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -444,13 +451,10 @@ chunk_outputs_kernel(ChunkArgs p) {
   for (int i = 0; i < NT; ++i)
 #pragma unroll
     for (int e = 0; e < 4; ++e) O[i][e] *= eA[e];
-  __syncthreads();                              // everybody is done with q, k and S_0
 #pragma unroll
   for (int i = 0; i < NT; ++i) {
-    const int e = tid + 256 * i, t = e / (4 * NT), c = 4 * (e % (4 * NT));
-    f32x4 v = {0.f, 0.f, 0.f, 0.f};
-    if (t < nt) v = load4(vp + (size_t)t * a.ld_v, v0 + c, a.dv, p.vec);
-    *reinterpret_cast<f32x4*>(sv + t * VS + c) = v;
+    const int e = tid + 256 * i;
+    *reinterpret_cast<f32x4*>(sv + (e / (4 * NT)) * VS + 4 * (e % (4 * NT))) = rv[i];
   }
   if (with_n) {
 #pragma unroll
@@ -535,6 +539,8 @@ mlstm_finish_kernel(const float* __restrict__ o, const float* __restrict__ nq, c
 
 MIE_EXPORT const char* matrix_state_last_error() { return g_mie_error; }
 
+constexpr long WIDE_FROM = 256;       // workgroups
+
 template <int NT>
 static int chunk_launch_nt(const ChunkArgs& p, int rows, hipStream_t s) {
   const ScanArgs& a = p.s;
@@ -560,7 +566,9 @@ static int scan_launch(const ScanArgs& a, int rows, int max_chunks, float* start
     const uintptr_t all = (uintptr_t)a.q | (uintptr_t)a.k | (uintptr_t)a.v | (uintptr_t)starts;
     const int vec = (all & 15) == 0 && a.ld_qk % 4 == 0 && a.ld_v % 4 == 0 && a.d % 4 == 0 && a.dv % 4 == 0;
     ChunkArgs p{a, max_chunks, vec, starts, n_starts, ends};
-    return a.dv <= 64 ? chunk_launch_nt<4>(p, rows, s) : chunk_launch_nt<8>(p, rows, s);
+    // 128 columns a workgroup where that still gives every compute unit one (the scores are then made half as often)
+    const bool wide = a.dv > 64 && (long)rows * max_chunks * a.H * ((a.dv + 127) / 128) >= WIDE_FROM;
+    return wide ? chunk_launch_nt<8>(p, rows, s) : chunk_launch_nt<4>(p, rows, s);
   }
   if (a.d > 1024) MIE_FAIL("matrix_scan: states of %d rows (at most 1024)", a.d);
   const int tiles = (a.dv + 63) / 64;

@@ -105,6 +105,52 @@ short_conv_kernel(const float* __restrict__ x, long ldx, const float* __restrict
   }
 }
 
+// The same for steps with rows of many tokens: a thread a channel of 16 tokens, the last inputs carried along (every number is
+// read once); the tail is only read.
+template <int KT>
+__global__ void __launch_bounds__(256)
+short_conv_tile_kernel(const float* __restrict__ x, long ldx, const float* __restrict__ taps, const float* __restrict__ bias,
+                       const float* __restrict__ tail, const int* __restrict__ token_row, const int* __restrict__ row_start,
+                       const int* __restrict__ slots, float* __restrict__ u, int tokens, int C, int act) {
+  constexpr int TT = 16, U = 4, keep = KT - 1;
+  const int c = blockIdx.y * 256 + threadIdx.x;
+  if (c >= C) return;
+  const int t_first = blockIdx.x * TT, t_end = t_first + TT < tokens ? t_first + TT : tokens;
+  float tp[KT], win[keep];
+#pragma unroll
+  for (int k = 0; k < KT; ++k) tp[k] = taps[(size_t)c * KT + k];
+  const float b = bias ? bias[c] : 0.f;
+#pragma unroll
+  for (int g = 0; g < TT; g += U) {
+    if (t_first + g >= t_end) break;
+    float in[U];
+#pragma unroll
+    for (int i = 0; i < U; ++i) in[i] = x[(size_t)(t_first + g + i < t_end ? t_first + g + i : t_end - 1) * ldx + c];
+#pragma unroll
+    for (int i = 0; i < U; ++i) {
+      const int t = t_first + g + i;
+      if (t >= t_end) break;
+      const int r = token_row[t], j = t - row_start[r];
+      if (g + i == 0 || j == 0) {               // the inputs before this token: of its row, or from the tail
+        const float* __restrict__ tl = tail + (size_t)slots[r] * keep * C;
+#pragma unroll
+        for (int k = 0; k < keep; ++k) {
+          const int back = keep - k;
+          win[k] = back <= j ? x[(size_t)(t - back) * ldx + c] : tl[(size_t)(keep + j - back) * C + c];
+        }
+      }
+      float acc = b;
+#pragma unroll
+      for (int k = 0; k < keep; ++k) acc = fmaf(tp[k], win[k], acc);
+      acc = fmaf(tp[keep], in[i], acc);
+#pragma unroll
+      for (int k = 0; k + 1 < keep; ++k) win[k] = win[k + 1];
+      win[keep - 1] = in[i];
+      u[(size_t)t * C + c] = mie_act(acc, act);
+    }
+  }
+}
+
 // the row's last K - 1 inputs (old tail, then this step's x), oldest first, into tail[slot]; a thread a (row, channel)
 __global__ void __launch_bounds__(256)
 conv_tail_move_kernel(const float* __restrict__ x, long ldx, float* __restrict__ tail, const int* __restrict__ row_start,
@@ -318,6 +364,18 @@ MIE_EXPORT int mie_short_conv(const float* x, long ldx, const float* taps, const
   if (act < MIE_ACT_NONE || act > MIE_ACT_RELU2) MIE_FAIL("short_conv: activation code %d", act);
   if (!x || !taps || !tail || !token_row || !row_start || !slots || !u) MIE_FAIL("short_conv: operands");
   int by = (C + 255) / 256;
+  if (tokens >= 64 && !move_tail && K >= 2 && K <= 4) {
+    const dim3 grid((tokens + 15) / 16, by);
+#define SCT(K_)                                                                                                                  \
+  hipLaunchKernelGGL(short_conv_tile_kernel<K_>, grid, dim3(256), 0, s, x, ldx, taps, bias, tail, token_row, row_start, slots, u, \
+                     tokens, C, act)
+    if (K == 2) SCT(2);
+    else if (K == 3) SCT(3);
+    else SCT(4);
+#undef SCT
+    MIE_CHECK_LAUNCH("short_conv (tiles)");
+    return 0;
+  }
   by = by > 64 ? 64 : by;
 #define SC(K_)                                                                                                              \
   hipLaunchKernelGGL(short_conv_kernel<K_>, dim3(tokens, by), dim3(256), 0, s, x, ldx, taps, bias, tail, token_row, row_start, \
