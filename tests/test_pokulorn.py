@@ -572,11 +572,11 @@ def test_batched_rows_equal_rows_alone():
         assert float((got[key] - row).abs().max()) < 1e-5 * float(row.abs().max())
 
 
-def generate(name, device, dtype, **engine):
+def generate(name, device, dtype, lengths=(9, 30, 2, 17, 23), budget=32, blocks=24, **engine):
     from mini_inference_engine_amd import LLMEngine, SamplingParams
     raw, cfg, weights = make(name, torch.float32 if dtype == "float32" else torch.bfloat16, sharp=dtype == "float32")
-    prompts = list(trace_util.random_prompts(raw["vocab"], [9, 30, 2, 17, 23], seed=4).values())
-    ecfg = EngineConfig(num_blocks=24, max_num_seqs=3, max_num_batched_tokens=32, max_model_len=128, **engine)
+    prompts = list(trace_util.random_prompts(raw["vocab"], list(lengths), seed=4).values())
+    ecfg = EngineConfig(num_blocks=blocks, max_num_seqs=3, max_num_batched_tokens=budget, max_model_len=max(128, max(lengths) + 32), **engine)
     kw = dict(device="cpu", backend=TorchBackend(torch.float32)) if device == "cpu" else {}
     eng = LLMEngine(cfg, ecfg, dtype=dtype, verbose=False, weights=weights, **kw)
     outs = eng.generate(prompts, SamplingParams(max_tokens=30, ignore_eos=True))          # through a window's edge
@@ -760,7 +760,7 @@ def test_kept_first_keys_and_head_sink_kernels(hip, dtype):
     ops, g = hip[dtype], torch.Generator().manual_seed(35)
     rows = [(0, 1), (5, 1), (23, 1), (63, 1), (64, 1), (200, 1), (700, 1), (0, 50), (17, 31), (63, 2), (100, 130), (0, 300), (400, 70)]
     for (Hq, Hkv, P, window, keep, sinks) in ((6, 2, 16, 24, 3, True), (3, 3, 32, 16, 20, True), (4, 1, 16, 40, 1, False), (2, 2, 48, 1, 66, True),
-                                              (8, 2, 64, 100, 130, True), (4, 4, 128, 33, 32, False), (16, 4, 64, 136, 64, True), (8, 4, 64, None, 0, True),
+                                              (8, 2, 64, 100, 130, True), (4, 4, 128, 33, 32, False), (16, 4, 64, 140, 64, True), (8, 4, 64, None, 0, True),
                                               (4, 2, 256, 50, 9, True), (4, 2, 64, 50, 0, True)):
         case = AttentionCase(rows, Hkv, P, dtype, g)
         q = _rand((case.num_tokens, Hq * P), dtype, g)
@@ -825,6 +825,14 @@ def test_long_prompts_in_chunks_of_the_recurrences(dtype):
 def test_greedy_generation_through_the_engine(dtype):
     eng = generate("A", "cuda", dtype)
     assert eng.num_graph_steps > 0, "decode steps run as captured graphs"
+
+
+@pytest.mark.gpu
+def test_captured_prompt_portions_run_the_recurrences_in_chunks():
+    """Prompts in portions of exactly the step's budget of 128 tokens: the captured step of such a portion is replayed for
+    portion after portion of several requests, each going on from its own states."""
+    eng = generate("D", "cuda", "bfloat16", lengths=(256, 384, 130, 256), budget=128, blocks=80)
+    assert eng.num_graph_steps > 0 and eng.runner.portion_graphs[-1].tokens == 128
 
 
 # --------------------------------------------------------------------------------------------- the command line
