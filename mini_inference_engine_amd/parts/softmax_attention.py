@@ -100,6 +100,11 @@ class SoftmaxAttention(Mixer):
         self.share_values, self.take_values = share_values, take_values
         if (share_values or take_values) and (self.values_from_keys or (share_values and take_values)):
             raise ValueError("a layer leaves its own values or takes another's, and projects them itself")
+        self.has_taps = self.conv is not None
+        if self.conv is None and (share_values or take_values or (position is not None and position.magnitude != 1.0)):
+            if bias or head_temperature or position_temperature is not None or (qk_norm and not self.norm_per_head):
+                raise ValueError("a scaled rotation and shared values are built with norms head by head, without biases and temperatures")
+            self.conv = 1           # built for convolved projections only: one tap of one leaves them as they are
         self.taps = self.value_mix = None
         self.mix = 0.0
         self.float32_output = bool(float32_output)
@@ -141,7 +146,7 @@ class SoftmaxAttention(Mixer):
         if self.qk_norm:
             specs += [ParamSpec.single("q_norm", name("q_norm"), (self.dim if self.norm_per_head else H * self.dim,), init="scale"),
                       ParamSpec.single("k_norm", name("k_norm"), (self.dim if self.norm_per_head else G * self.dim,), init="scale")]
-        if self.conv is not None:
+        if self.has_taps:
             specs.append(ParamSpec.stacked("taps", [(name("q_conv"), (H * self.dim, self.conv)), (name("k_conv"), (G * self.dim, self.conv)),
                                                     (name("v_conv"), (G * self.vdim, self.conv))]))
         if self.head_sink:
@@ -179,6 +184,8 @@ class SoftmaxAttention(Mixer):
         for attr in ("temperature", "q_norm", "k_norm", "taps") + (("sink",) if self.head_sink else ()):     # 32-bit whatever the checkpoint stores
             if getattr(self, attr, None) is not None:
                 setattr(self, attr, getattr(self, attr).float().contiguous())
+        if self.conv is not None and not self.has_taps:
+            self.taps = torch.ones((self.channels, 1), dtype=torch.float32, device=self.w_in.device)
         if self.value_mix is not None:
             self.mix = float(self.value_mix)
         if self.b_in is not None:       # one number a column of the product's sums, zeros for the columns nobody reads

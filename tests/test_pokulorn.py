@@ -92,7 +92,7 @@ B_MIX = att(4, 1, 24, vdim=8, window=40, keep=1, v_mix=True, conv=5)
 CFG_B = model(150, 48, 1e-3, [layer("attention", B_PLAIN, dense(56, 0.7)),
                               layer("parallel", pair(att(2, 2, 16, conv=3, scale=0.3), ssm(4, 16, 12, groups=4, conv=2, norm_groups=1), 2.0, 0.25), None),
                               layer("attention", B_MIX, dense(40)),
-                              layer("attention", att(4, 4, 16, v_mix=False, conv=None, rotation=rot(4)), dense(40)),   # no window, no convolution
+                              layer("attention", att(4, 4, 16, v_mix=False, conv=None, rotation=rot(4, factor=3.0)), dense(40)),   # no window, no convolution
                               layer("attention", B_MIX, None)])
 # sizes the kernels' vector paths do not like: nothing a multiple of 8, an odd vocabulary, one head of everything
 CFG_C = model(101, 70, 1e-6, [layer("parallel", pair(att(3, 1, 10, vdim=14, conv=1, rotation=rot(6, factor=2.0)), ssm(5, 6, 7, conv=3, norm_groups=3), 1.0, 1.0), dense(50, 9.0)),
@@ -220,7 +220,7 @@ def test_config_round_trip_and_registry(tmp_path):
     a, b, c = (PokulornConfig.from_dict(CONFIGS[n][0]) for n in "ABC")
     assert a.first_value_layer() == 0 and b.first_value_layer() == 2 and c.first_value_layer() == 2
     assert a.layers[0].mixer.vdim == 24 and a.layers[0].mixer.keep_first == 3 and a.layers[3].mlp is None
-    assert b.layers[3].mixer.window is None and b.layers[3].mixer.taps is None and b.layers[3].mixer.rot.scaling is None
+    assert b.layers[3].mixer.window is None and b.layers[3].mixer.taps is None and b.layers[0].mixer.rot.scaling is None
     assert c.layers[3].mixer.vdim == 5 and c.layers[4].mixer.keep_first == 0
 
 
@@ -334,6 +334,7 @@ MECHANISMS = {
     "attention-window-of-one": one_layer("attention", att(2, 1, 8, window=1, keep=1, conv=2), None),
     "attention-window-keeps-nothing": one_layer("attention", att(2, 1, 8, window=7, keep=0), None),
     "attention-no-convolution": one_layer("attention", att(3, 1, 8, conv=None, rotation=rot(8), window=9, keep=17), None),
+    "attention-no-convolution-values-mixed": model(50, 32, 1e-5, [layer("attention", att(2, 1, 8, v_mix=True, conv=None, rotation=rot(8)), None)] * 2),
     "attention-one-tap": one_layer("attention", att(1, 1, 24, vdim=40, conv=1, rotation=rot(6, factor=3.0)), None),
     "values-mixed": model(50, 32, 1e-5, [layer("attention", att(2, 1, 8, vdim=12, v_mix=True, window=5, keep=1), None),
                                          layer("attention", att(4, 1, 16, vdim=12, v_mix=True, conv=2), None)]),
