@@ -32,8 +32,8 @@ class YarnSpec:
 
 @dataclass(frozen=True)
 class YarnRotarySpec:
-    """Pairs (i, i + dims / 2) of the first ``dims`` numbers of a head turn by base^(-2i / dims) a position, stretched by
-    parts where ``scaling`` is given."""
+    """The first ``dims`` numbers of a head turn in pairs (which two are a pair is the design's), pair i by base^(-2i / dims) a
+    position, stretched by parts where ``scaling`` is given."""
     base: float
     dims: int
     scaling: YarnSpec | None = None

@@ -48,7 +48,8 @@ struct ProjectionSums {
 // KEEP: beside the window the row sees its request's first ``keep`` keys.  The blocks that hold them come before the
 // window's in the order the splits and waves walk: index x of that order is key x up to the end of the kept blocks, key
 // x + gap behind it, gap a whole number of blocks.
-template <int NW, bool FROM_SUMS, bool SIG = false, bool DB = false, bool KEEP = false>
+// CHUNK: the softmax over the keys of the row's own chunk of positions (from floor(position / chunk) chunk on).
+template <int NW, bool FROM_SUMS, bool SIG = false, bool DB = false, bool KEEP = false, bool CHUNK = false>
 __global__ void __launch_bounds__(NW * 64)
 decode_attention_kernel(const bf16* __restrict__ q, long q_stride, bf16* k_cache, bf16* v_cache,
                         bf16* __restrict__ out, float* __restrict__ o_part,
@@ -59,6 +60,7 @@ decode_attention_kernel(const bf16* __restrict__ q, long q_stride, bf16* k_cache
                         const float* __restrict__ dist_bias, int dist_n, int keep, const float* __restrict__ head_sinks) {
   static_assert(!(DB && (SIG || FROM_SUMS)), "the distance bias is built for the softmax over finished queries");
   static_assert(!(KEEP && (SIG || FROM_SUMS || DB)), "kept first keys are built for the plain softmax over finished queries");
+  static_assert(!(CHUNK && (SIG || FROM_SUMS || DB || KEEP)), "chunks are built for the plain softmax over finished queries, and for sigmoids");
   __shared__ float s_m[NW][16], s_l[NW][16], s_M[16], s_L[16];
   __shared__ float s_o[NW][16][D + 1];
   __shared__ __align__(16) bf16 s_q[FROM_SUMS ? 16 : 1][D];
@@ -119,7 +121,7 @@ decode_attention_kernel(const bf16* __restrict__ q, long q_stride, bf16* k_cache
   KeyBlock b0, b1;
   const int pos_raw = positions[b];
   int begin0 = s * partition;               // the split's first key when there is no window
-  if (AHEAD && window <= 0 && (!SIG || chunk <= 0)) load_block(b0, begin0 + BLOCK_KEYS * wave);
+  if (AHEAD && !CHUNK && window <= 0 && (!SIG || chunk <= 0)) load_block(b0, begin0 + BLOCK_KEYS * wave);
 
   const int pos = pos_raw;
   if (FROM_SUMS) {
@@ -168,8 +170,10 @@ decode_attention_kernel(const bf16* __restrict__ q, long q_stride, bf16* k_cache
   // DB: the lane's head's row of the distance table (entries already times log2 e)
   const float* __restrict__ db_row = DB ? dist_bias + (size_t)head * dist_n : nullptr;
   float sg_c1 = 0.f, sg_c2 = 0.f, sg_c3 = 0.f;
-  if constexpr (SIG) {
+  if constexpr (SIG || CHUNK) {
     if (chunk > 0 && pos / chunk * chunk > lo) lo = pos / chunk * chunk;
+  }
+  if constexpr (SIG) {
     const float hb = head_bias ? head_bias[head] : 0.f;
     const float L2E = 1.4426950408889634f;
     if (softcap > 0.f) {
@@ -337,7 +341,7 @@ decode_attention_kernel(const bf16* __restrict__ q, long q_stride, bf16* k_cache
   constexpr int STEP = BLOCK_KEYS * NW;     // keys from one block of a wave to its next
   const int first = begin + BLOCK_KEYS * wave;
   if (AHEAD) {
-    if (window > 0 || (SIG && chunk > 0)) load_block(b0, key_of(first));  // with a window the split's start had to wait for the row's length
+    if (CHUNK || window > 0 || (SIG && chunk > 0)) load_block(b0, key_of(first));  // with a window the split's start had to wait for the row's length
     const int part_end = begin + partition;   // nothing is asked for beyond the split's own keys
     for (int blk = first; blk < end; blk += 2 * STEP) {
       if (blk + STEP < part_end) load_block(b1, key_of(blk + STEP));           // in flight while block 0 is computed
@@ -498,7 +502,18 @@ static int decode_attention_launch(const void* q, long q_stride, const void* k_c
   bf16* kc = (bf16*)const_cast<void*>(k_cache);
   bf16* vc = (bf16*)const_cast<void*>(v_cache);
   const bool whole = num_splits == 1 && NW_WHOLE != NW_SPLIT && (long)rows * Hkv * head_tiles < NW_WHOLE_BELOW;
-  if (keep > 0 && whole)
+  if (chunk > 0 && !sigmoid && (keep > 0 || dist_bias)) MIE_FAIL("decode_attention: chunks beside kept keys or a distance bias are not built");
+  if (chunk > 0 && !sigmoid && whole)
+    hipLaunchKernelGGL((decode_attention_kernel<NW_WHOLE, false, false, false, false, true>), grid, dim3(NW_WHOLE * 64), 0, stream,
+                       (const bf16*)q, q_stride, kc, vc, (bf16*)out, o_part, lse_part, block_tables, max_blocks, positions, Hq, Hkv,
+                       head_tiles, page, scale * 1.4426950408889634f, window, partition, num_splits, ProjectionSums{}, sink_log2, chunk, 0.f,
+                       (const float*)nullptr, (const float*)nullptr, 0, 0, head_sinks);
+  else if (chunk > 0 && !sigmoid)
+    hipLaunchKernelGGL((decode_attention_kernel<NW_SPLIT, false, false, false, false, true>), grid, dim3(NW_SPLIT * 64), 0, stream,
+                       (const bf16*)q, q_stride, kc, vc, (bf16*)out, o_part, lse_part, block_tables, max_blocks, positions, Hq, Hkv,
+                       head_tiles, page, scale * 1.4426950408889634f, window, partition, num_splits, ProjectionSums{}, sink_log2, chunk, 0.f,
+                       (const float*)nullptr, (const float*)nullptr, 0, 0, head_sinks);
+  else if (keep > 0 && whole)
     hipLaunchKernelGGL((decode_attention_kernel<NW_WHOLE, false, false, false, true>), grid, dim3(NW_WHOLE * 64), 0, stream, (const bf16*)q,
                        q_stride, kc, vc, (bf16*)out, o_part, lse_part, block_tables, max_blocks, positions, Hq, Hkv, head_tiles, page,
                        scale * 1.4426950408889634f, window, partition, num_splits, ProjectionSums{}, sink_log2, 0, 0.f,
@@ -701,4 +716,17 @@ MIE_EXPORT int mie_decode_attention_kept(const void* q, long q_stride, const voi
   return decode_attention_launch(q, q_stride, k_cache, v_cache, out, o_part, lse_part, block_tables, max_blocks, positions,
                                  rows, Hq, Hkv, head_dim, page, scale, window, partition, num_splits, -INFINITY, stream, false,
                                  0, 0.f, nullptr, nullptr, 0, keep, head_sinks);
+}
+
+// The softmax over the keys of the row's own chunk of positions, from floor(position / chunk) chunk on (and over the last
+// ``window`` of them, if that is not 0).
+MIE_EXPORT int mie_decode_attention_chunked(const void* q, long q_stride, const void* k_cache, const void* v_cache, void* out,
+                                            float* o_part, float* lse_part, const int* block_tables, int max_blocks,
+                                            const int* positions, int rows, int Hq, int Hkv, int head_dim, int page,
+                                            float scale, int window, int partition, int num_splits, int chunk,
+                                            hipStream_t stream) {
+  if (chunk < 1) MIE_FAIL("decode_attention_chunked: chunks of %d positions", chunk);
+  return decode_attention_launch(q, q_stride, k_cache, v_cache, out, o_part, lse_part, block_tables, max_blocks, positions,
+                                 rows, Hq, Hkv, head_dim, page, scale, window, partition, num_splits, -INFINITY, stream, false,
+                                 chunk);
 }

@@ -7,8 +7,9 @@
 // qkv_finish: one workgroup a token.  Queries go out as [T, Hq, P], keys to k_cache [pages, Hkv, page, P], values
 // to v_cache [pages, Hkv, P, page] (transposed within a page), zeros beyond dim / vdim.  Everything is computed in
 // 32-bit from the sums and rounded once on the way out.
-// qkv_conv_finish: the same for projections that first pass a short causal convolution over time (with norms head by head,
-// halves turned, a factor on cosines and sines, values left for or mixed with another layer's).
+// qkv_conv_finish: the same for projections that first pass a short causal convolution over time (with biases before it, norms
+// head by head before the rotation or, without weights, after it, either pairing turned, a factor on cosines and sines, values
+// left for or mixed with another layer's).
 // head_gate:  o[t, h, :] *= sigmoid(gate[t, h]).
 // gate_heads: out[t, h vdim + d] = scale * o[t, h P + d] * sigmoid(gate[t, h vdim + d]), d < vdim.
 #include "common.hpp"
@@ -118,12 +119,14 @@ qkv_finish_kernel(FinishArgs a) {
 // ---- projections through a short convolution
 struct ConvFinishArgs {
   const float* sums; long ld; int col;                      // queries, keys, values side by side from column ``col`` on
+  const float* col_bias;        // [C], added to the inputs of the convolution (the tail holds biased inputs), or null
   const float* taps;            // [C, K], C = (Hq + Hkv) dim + Hkv vdim in that order
   float* tail;                  // [slots, K - 1, C]: the row's last inputs, oldest first
   const int* token_row; const int* row_start; const int* state_slots;
   int K, move_tail;             // move_tail: every row is one token, and the waves move the tail on themselves
   const float* q_norm; const float* k_norm; float eps;      // dim numbers each, or null
-  const float* inv_freq; int nf; float rot_scale;
+  int norm_turned;              // no weights: heads over their root mean square after the rotation
+  const float* inv_freq; int nf, layout; float rot_scale;
   const int* positions; const int* slots;
   float* values_out; const float* mix_other; float mix;     // values as projected / (1 - mix) v + mix * other
   void* q_out; void* k_cache; void* v_cache;
@@ -152,9 +155,11 @@ qkv_conv_finish_kernel(ConvFinishArgs a) {
     const int n = is_v ? a.vdim : a.dim;
     const int c0 = is_q ? h * a.dim : is_v ? (a.Hq + a.Hkv) * a.dim + h * a.vdim : (a.Hq + h) * a.dim;
     float ss = 0.f;
+    const float grown = a.norm_turned ? a.rot_scale * a.rot_scale : 1.f;      // what the rotation does to a pair's sum of squares
     for (int d = lane; d < n; d += 64) {
       const int c = c0 + d;
       const float* __restrict__ x = a.sums + (size_t)t * a.ld + a.col + c;
+      const float b = a.col_bias ? a.col_bias[c] : 0.f;
       float acc = 0.f;
       if constexpr (KT > 0) {
         float in[KT];
@@ -162,7 +167,7 @@ qkv_conv_finish_kernel(ConvFinishArgs a) {
         for (int i = 0; i < KT; ++i) {          // tokens t - K + 1 .. t
           const int back = KT - 1 - i;
           const float* src = back <= j ? x - (long)back * a.ld : tl + (size_t)(keep + j - back) * a.C + c;
-          in[i] = *src;
+          in[i] = *src + (back <= j ? b : 0.f);
         }
 #pragma unroll
         for (int i = 0; i < KT; ++i) acc = fmaf(a.taps[(size_t)c * KT + i], in[i], acc);
@@ -173,13 +178,13 @@ qkv_conv_finish_kernel(ConvFinishArgs a) {
       } else {
         for (int i = 0; i < K; ++i) {
           const int back = K - 1 - i;
-          acc = fmaf(a.taps[(size_t)c * K + i], back <= j ? x[-(long)back * a.ld] : tl[(size_t)(keep + j - back) * a.C + c], acc);
+          acc = fmaf(a.taps[(size_t)c * K + i], back <= j ? x[-(long)back * a.ld] + b : tl[(size_t)(keep + j - back) * a.C + c], acc);
         }
         if (a.move_tail)
-          for (int i = 0; i < keep; ++i) tl[(size_t)i * a.C + c] = i + 1 < keep ? tl[(size_t)(i + 1) * a.C + c] : x[0];
+          for (int i = 0; i < keep; ++i) tl[(size_t)i * a.C + c] = i + 1 < keep ? tl[(size_t)(i + 1) * a.C + c] : x[0] + b;
       }
       mine[d] = acc;
-      ss = fmaf(acc, acc, ss);
+      ss = fmaf(d < 2 * a.nf ? grown * acc : acc, acc, ss);
     }
     __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");      // the wave's lanes read one another's numbers below
     __builtin_amdgcn_wave_barrier();
@@ -197,19 +202,20 @@ qkv_conv_finish_kernel(ConvFinishArgs a) {
       }
     } else {
       const float* __restrict__ w = is_q ? a.q_norm : a.k_norm;
-      const float rms = w ? 1.0f / sqrtf(wave_sum(ss) / (float)n + a.eps) : 1.f;
+      const float rms = w || a.norm_turned ? 1.0f / sqrtf(wave_sum(ss) / (float)n + a.eps) : 1.f;
       TO* __restrict__ dst = is_q ? (TO*)a.q_out + ((size_t)t * a.Hq + h) * a.P
                                   : (TO*)a.k_cache + ((pg * a.Hkv + h) * a.page + off) * a.P;
       for (int i = lane; i < a.nf; i += 64) {
         float c, s, o1, o2;
         sincosf(pos * a.inv_freq[i], &s, &c);
-        const float x1 = w ? mine[i] * rms * w[i] : mine[i], x2 = w ? mine[i + a.nf] * rms * w[i + a.nf] : mine[i + a.nf];
+        const int d1 = a.layout == LAYOUT_INTERLEAVED ? 2 * i : i, d2 = a.layout == LAYOUT_INTERLEAVED ? 2 * i + 1 : i + a.nf;
+        const float x1 = w ? mine[d1] * rms * w[d1] : mine[d1] * rms, x2 = w ? mine[d2] * rms * w[d2] : mine[d2] * rms;
         rotate_pair(x1, x2, c * a.rot_scale, s * a.rot_scale, o1, o2);
-        dst[i] = from_float<TO>(o1);
-        dst[i + a.nf] = from_float<TO>(o2);
+        dst[d1] = from_float<TO>(o1);
+        dst[d2] = from_float<TO>(o2);
       }
       for (int d = 2 * a.nf + lane; d < a.P; d += 64)
-        dst[d] = from_float<TO>(d < n ? (w ? mine[d] * rms * w[d] : mine[d]) : 0.f);
+        dst[d] = from_float<TO>(d < n ? (w ? mine[d] * rms * w[d] : mine[d] * rms) : 0.f);
     }
     __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");      // before the next head's numbers replace these
     __builtin_amdgcn_wave_barrier();
@@ -250,13 +256,16 @@ qkv_conv_finish_tile_kernel(ConvFinishArgs a, int tokens) {
     const int n = is_v ? a.vdim : a.dim;
     const int c0 = is_q ? h * a.dim : is_v ? (a.Hq + a.Hkv) * a.dim + h * a.vdim : (a.Hq + h) * a.dim;
     const float* __restrict__ w = is_q ? a.q_norm : a.k_norm;
-    float tp[E][KT], win[E][keep], wn[E];
+    const bool normed = w || a.norm_turned;
+    const float grown = a.norm_turned ? a.rot_scale * a.rot_scale : 1.f;      // what the rotation does to a pair's sum of squares
+    float tp[E][KT], win[E][keep], wn[E], bi[E];
     int ch[E];                                                // the lane's channels, clamped into the head
 #pragma unroll
     for (int e = 0; e < E; ++e) {
       const int d = lane + 64 * e;
       ch[e] = c0 + (d < n ? d : n - 1);
       wn[e] = !is_v && w && d < n ? w[d] : 1.f;
+      bi[e] = a.col_bias ? a.col_bias[ch[e]] : 0.f;
 #pragma unroll
       for (int k = 0; k < KT; ++k) tp[e][k] = a.taps[(size_t)ch[e] * KT + k];
     }
@@ -267,7 +276,7 @@ qkv_conv_finish_tile_kernel(ConvFinishArgs a, int tokens) {
       for (int u = 0; u < U; ++u) {
         const int t = t_first + g + u < t_end ? t_first + g + u : t_end - 1;
 #pragma unroll
-        for (int e = 0; e < E; ++e) x[u][e] = a.sums[(size_t)t * a.ld + a.col + ch[e]];
+        for (int e = 0; e < E; ++e) x[u][e] = a.sums[(size_t)t * a.ld + a.col + ch[e]] + bi[e];
       }
 #pragma unroll
       for (int u = 0; u < U; ++u) {
@@ -280,7 +289,7 @@ qkv_conv_finish_tile_kernel(ConvFinishArgs a, int tokens) {
 #pragma unroll
             for (int i = 0; i < keep; ++i) {
               const int back = keep - i;
-              win[e][i] = back <= j ? a.sums[(size_t)(t - back) * a.ld + a.col + ch[e]] : tl[(size_t)(keep + j - back) * a.C + ch[e]];
+              win[e][i] = back <= j ? a.sums[(size_t)(t - back) * a.ld + a.col + ch[e]] + bi[e] : tl[(size_t)(keep + j - back) * a.C + ch[e]];
             }
         }
         ss[u] = 0.f;
@@ -294,7 +303,7 @@ qkv_conv_finish_tile_kernel(ConvFinishArgs a, int tokens) {
           for (int i = 0; i + 1 < keep; ++i) win[e][i] = win[e][i + 1];
           win[e][keep - 1] = x[u][e];
           y[u][e] = lane + 64 * e < n ? acc : 0.f;
-          ss[u] = fmaf(y[u][e], y[u][e], ss[u]);
+          ss[u] = fmaf(lane + 64 * e < 2 * a.nf ? grown * y[u][e] : y[u][e], y[u][e], ss[u]);
         }
       }
       if (is_v) {
@@ -329,7 +338,7 @@ qkv_conv_finish_tile_kernel(ConvFinishArgs a, int tokens) {
         }
         continue;
       }
-      if (w) {
+      if (normed) {
 #pragma unroll
         for (int o = 32; o > 0; o >>= 1)
 #pragma unroll
@@ -337,7 +346,7 @@ qkv_conv_finish_tile_kernel(ConvFinishArgs a, int tokens) {
       }
 #pragma unroll
       for (int u = 0; u < U; ++u) {
-        const float rms = w ? 1.0f / sqrtf(ss[u] / (float)n + a.eps) : 1.f;
+        const float rms = normed ? 1.0f / sqrtf(ss[u] / (float)n + a.eps) : 1.f;
 #pragma unroll
         for (int e = 0; e < E; ++e) {
           y[u][e] *= rms * wn[e];
@@ -359,9 +368,9 @@ qkv_conv_finish_tile_kernel(ConvFinishArgs a, int tokens) {
             if (d < P) {
               float o = y[u][e];
               if (d < 2 * a.nf) {
-                const bool low = d < a.nf;
-                const int f = low ? d : d - a.nf;
-                const float c = cs[(g + u) * a.nf + f], s = sn[(g + u) * a.nf + f], other = mine[u * P + (low ? d + a.nf : f)];
+                const bool half = a.layout == LAYOUT_HALF, low = half ? d < a.nf : (d & 1) == 0;
+                const int f = half ? (low ? d : d - a.nf) : d >> 1, partner = half ? (low ? d + a.nf : f) : d ^ 1;
+                const float c = cs[(g + u) * a.nf + f], s = sn[(g + u) * a.nf + f], other = mine[u * P + partner];
                 o = low ? fmaf(o, c, -(other * s)) : fmaf(o, c, other * s);
               }
               dst[d] = from_float<TO>(o);
@@ -438,11 +447,12 @@ MIE_EXPORT int mie_head_gate(void* o, int dtype, const float* gate, long ldg, in
 
 // taps [C, K] and tail [slots, max(1, K - 1), C] float32, C = (Hq + Hkv) dim + Hkv vdim channels that lie side by side in the
 // sums from column col on.  move_tail: every row of the step is one token, and the tail moves on here; else the caller moves
-// it afterwards.  values_out, mix_other float32 [tokens, Hkv vdim] or null.
-MIE_EXPORT int mie_qkv_conv_finish(const float* sums, long ld, int col, const float* taps, float* tail, const int* token_row,
-                                   const int* row_start, const int* state_slots, int K, int move_tail, const float* q_norm,
-                                   const float* k_norm, float eps, const float* inv_freq, int nf, float rot_scale,
-                                   const int* positions, const int* slots, float* values_out, const float* mix_other, float mix,
+// it afterwards.  col_bias float32 [C] or null.  norm_turned: q_norm and k_norm are null, and heads are divided by their root
+// mean square after the rotation.  values_out, mix_other float32 [tokens, Hkv vdim] or null.
+MIE_EXPORT int mie_qkv_conv_finish(const float* sums, long ld, int col, const float* col_bias, const float* taps, float* tail,
+                                   const int* token_row, const int* row_start, const int* state_slots, int K, int move_tail,
+                                   const float* q_norm, const float* k_norm, float eps, int norm_turned, const float* inv_freq, int nf,
+                                   int layout, float rot_scale, const int* positions, const int* slots, float* values_out, const float* mix_other, float mix,
                                    void* q_out, void* k_cache, void* v_cache, int dtype, int tokens, int Hq, int Hkv, int dim,
                                    int vdim, int P, int page, hipStream_t s) {
   if (tokens <= 0) return 0;
@@ -450,11 +460,13 @@ MIE_EXPORT int mie_qkv_conv_finish(const float* sums, long ld, int col, const fl
     MIE_FAIL("qkv_conv_finish: %d / %d heads of %d (values %d) in %d (at most 1024), page %d", Hq, Hkv, dim, vdim, P, page);
   if (2 * nf > dim || nf < 0 || (nf > 0 && !inv_freq)) MIE_FAIL("qkv_conv_finish: %d turned pairs in heads of %d", nf, dim);
   if (K < 1 || !taps || !tail || !token_row || !row_start || !state_slots) MIE_FAIL("qkv_conv_finish: %d taps and their operands", K);
+  if (layout != LAYOUT_INTERLEAVED && layout != LAYOUT_HALF) MIE_FAIL("qkv_conv_finish: layout code %d", layout);
+  if (norm_turned && (q_norm || k_norm)) MIE_FAIL("qkv_conv_finish: norms after the rotation have no weights");
   const int C = (Hq + Hkv) * dim + Hkv * vdim;
   if (ld < (long)col + C) MIE_FAIL("qkv_conv_finish: %d channels from column %d in rows of %ld", C, col, ld);
   const int row_floats = (dim > vdim ? dim : vdim);
-  ConvFinishArgs a{sums, ld, col, taps, tail, token_row, row_start, state_slots, K, move_tail, q_norm, k_norm, eps, inv_freq, nf,
-                   rot_scale, positions, slots, values_out, mix_other, mix, q_out, k_cache, v_cache, Hq, Hkv, dim, vdim, P, page, C,
+  ConvFinishArgs a{sums, ld, col, col_bias, taps, tail, token_row, row_start, state_slots, K, move_tail, q_norm, k_norm, eps, norm_turned,
+                   inv_freq, nf, layout, rot_scale, positions, slots, values_out, mix_other, mix, q_out, k_cache, v_cache, Hq, Hkv, dim, vdim, P, page, C,
                    row_floats};
   // rows of many tokens: 16 tokens a workgroup (the angles' table of a workgroup has to fit beside the heads)
   if (tokens >= 64 && !move_tail && K >= 2 && K <= 4 && P <= 256 && nf <= 128) {

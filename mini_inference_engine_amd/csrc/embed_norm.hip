@@ -1,16 +1,17 @@
 // Token embedding into the 32-bit residual stream, and the residual add fused with RMSNorm.
 //
-// embedding:    stream[t, :] = float(table[ids[t], :]) * scale
+// embedding:    stream[t, :] = float(table[ids[t], :]) * scale (and the same, rounded, into a second place)
+// stream_copy:  out[t, :] = stream[t, :] (+ float(x[t, :])) (+ x_bias), rounded once; the stream stays as it is
 // add_rmsnorm:  r = stream[row] (+ float(x[row]));  stream[row] = r (unless rows are gathered);
 //               y[row] = r * (1 / sqrt(mean(r^2) + eps)) * weight, rounded once to y's type.
 // One workgroup per row; the row's sum of squares is reduced in an order that depends only on
 // the row width, so a token's result does not depend on what else is in the batch.
 #include "common.hpp"
 
-template <typename TT>
+template <typename TT, typename TC>
 __global__ void embedding_kernel(const int* __restrict__ ids, const TT* __restrict__ table, float* __restrict__ out,
                                  int width, int vocab, const int* __restrict__ taken_from,
-                                 const int* __restrict__ earlier_tokens, float scale) {
+                                 const int* __restrict__ earlier_tokens, float scale, TC* __restrict__ copy, long ld_copy) {
   const int t = blockIdx.x;
   int id = ids[t];
   if (taken_from) {            // a token the host does not know yet: entry taken_from[t] of the tokens chosen last
@@ -20,7 +21,53 @@ __global__ void embedding_kernel(const int* __restrict__ ids, const TT* __restri
   id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);   // ids are validated on the host; never read outside
   const TT* src = table + (size_t)id * width;
   float* dst = out + (size_t)t * width;
-  for (int i = threadIdx.x; i < width; i += blockDim.x) dst[i] = to_float(src[i]) * scale;
+  for (int i = threadIdx.x; i < width; i += blockDim.x) {
+    const float v = to_float(src[i]) * scale;
+    dst[i] = v;
+    if (copy) copy[(size_t)t * ld_copy + i] = from_float<TC>(v);
+  }
+}
+
+template <typename TX, typename TO>
+__global__ void __launch_bounds__(256)
+stream_copy_kernel(const TX* __restrict__ x, const float* __restrict__ x_bias, const float* __restrict__ stream,
+                   TO* __restrict__ out, long ld_out, int width) {
+  const size_t row = (size_t)blockIdx.x * width;
+  TO* dst = out + (size_t)blockIdx.x * ld_out;
+  for (int i = blockIdx.y * 256 + threadIdx.x; i < width; i += gridDim.y * 256) {
+    float v = stream[row + i];
+    if (x) v += to_float(x[row + i]);
+    if (x_bias) v += x_bias[i];
+    dst[i] = from_float<TO>(v);
+  }
+}
+
+// the same, four numbers a thread
+template <typename TX, typename TO>
+__global__ void __launch_bounds__(256)
+stream_copy4_kernel(const TX* __restrict__ x, const float* __restrict__ x_bias, const float* __restrict__ stream,
+                    TO* __restrict__ out, long ld_out, int width) {
+  const size_t row = (size_t)blockIdx.x * width;
+  TO* dst = out + (size_t)blockIdx.x * ld_out;
+  struct alignas(4 * sizeof(TX)) InX { TX v[4]; };
+  struct alignas(4 * sizeof(TO)) Out { TO v[4]; };
+  for (int i = 4 * (blockIdx.y * 256 + threadIdx.x); i < width; i += 4 * gridDim.y * 256) {
+    const float4 s = *reinterpret_cast<const float4*>(stream + row + i);
+    float v[4] = {s.x, s.y, s.z, s.w};
+    if (x) {
+      const InX a = *reinterpret_cast<const InX*>(x + row + i);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] += to_float(a.v[e]);
+    }
+    if (x_bias) {
+      const float4 b = *reinterpret_cast<const float4*>(x_bias + i);
+      v[0] += b.x; v[1] += b.y; v[2] += b.z; v[3] += b.w;
+    }
+    Out o;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) o.v[e] = from_float<TO>(v[e]);
+    *reinterpret_cast<Out*>(dst + i) = o;
+  }
 }
 
 #define NORM_THREADS 256
@@ -165,22 +212,54 @@ MIE_EXPORT const char* embed_norm_last_error() { return g_mie_error; }
 
 // taken_from (or null) [tokens]: where >= 0, the token is earlier_tokens[taken_from[t]] instead of ids[t]
 // (a token chosen by the step before, which the host has not seen yet).
+// copy: a second place for the rows (null: none), of copy_dtype, rows ld_copy numbers apart
 MIE_EXPORT int mie_embedding(const int* ids, const void* table, int table_dtype, float* out, int tokens, int width,
-                             int vocab, const int* taken_from, const int* earlier_tokens, float scale,
-                             hipStream_t stream) {
+                             int vocab, const int* taken_from, const int* earlier_tokens, float scale, void* copy, int copy_dtype,
+                             long ld_copy, hipStream_t stream) {
   if (tokens <= 0) return 0;
   if (width <= 0 || vocab <= 0) MIE_FAIL("embedding: width %d, vocab %d", width, vocab);
   if (taken_from && !earlier_tokens) MIE_FAIL("embedding: taken_from without the tokens to take from");
+  if (copy && ld_copy < width) MIE_FAIL("embedding: rows of the copy %ld apart for width %d", ld_copy, width);
+  if (copy_dtype != MIE_F32 && copy_dtype != MIE_BF16) MIE_FAIL("embedding: copy dtype code %d", copy_dtype);
   dim3 grid(tokens), block(256);
-  if (table_dtype == MIE_F32)
-    hipLaunchKernelGGL(embedding_kernel<float>, grid, block, 0, stream, ids, (const float*)table, out, width, vocab,
-                       taken_from, earlier_tokens, scale);
-  else if (table_dtype == MIE_BF16)
-    hipLaunchKernelGGL(embedding_kernel<bf16>, grid, block, 0, stream, ids, (const bf16*)table, out, width, vocab,
-                       taken_from, earlier_tokens, scale);
+#define EMB(TT, TC)                                                                                                            \
+  hipLaunchKernelGGL((embedding_kernel<TT, TC>), grid, block, 0, stream, ids, (const TT*)table, out, width, vocab, taken_from, \
+                     earlier_tokens, scale, (TC*)copy, ld_copy)
+  if (table_dtype == MIE_F32 && copy_dtype == MIE_F32) EMB(float, float);
+  else if (table_dtype == MIE_F32) EMB(float, bf16);
+  else if (table_dtype == MIE_BF16 && copy_dtype == MIE_F32) EMB(bf16, float);
+  else if (table_dtype == MIE_BF16) EMB(bf16, bf16);
   else
     MIE_FAIL("embedding: table dtype code %d", table_dtype);
+#undef EMB
   MIE_CHECK_LAUNCH("embedding");
+  return 0;
+}
+
+// x [tokens, width] of x_dtype or null; x_bias float32 [width] or null; out of out_dtype, rows ld_out numbers apart
+MIE_EXPORT int mie_stream_copy(const void* x, int x_dtype, const float* x_bias, const float* stream_in, void* out, int out_dtype,
+                               long ld_out, int tokens, int width, hipStream_t stream) {
+  if (tokens <= 0) return 0;
+  if (width <= 0 || ld_out < width || !stream_in || !out) MIE_FAIL("stream_copy: width %d, rows %ld apart, or a null operand", width, ld_out);
+  const size_t esz = out_dtype == MIE_F32 ? 4 : 2, xsz = x_dtype == MIE_F32 ? 4 : 2;
+  const bool four = width % 4 == 0 && ld_out % 4 == 0 && (uintptr_t)stream_in % 16 == 0 && (uintptr_t)x_bias % 16 == 0 &&
+                    (uintptr_t)x % (4 * xsz) == 0 && (uintptr_t)out % (4 * esz) == 0;
+  int by = (width + (four ? 1023 : 255)) / (four ? 1024 : 256);
+  by = by > 16 ? 16 : by;
+#define SCP(TX, TO)                                                                                                              \
+  do {                                                                                                                           \
+    if (four) hipLaunchKernelGGL((stream_copy4_kernel<TX, TO>), dim3(tokens, by), dim3(256), 0, stream, (const TX*)x, x_bias,    \
+                                 stream_in, (TO*)out, ld_out, width);                                                            \
+    else hipLaunchKernelGGL((stream_copy_kernel<TX, TO>), dim3(tokens, by), dim3(256), 0, stream, (const TX*)x, x_bias, stream_in, \
+                            (TO*)out, ld_out, width);                                                                            \
+  } while (0)
+  if (x_dtype == MIE_F32 && out_dtype == MIE_F32) SCP(float, float);
+  else if (x_dtype == MIE_F32 && out_dtype == MIE_BF16) SCP(float, bf16);
+  else if (x_dtype == MIE_BF16 && out_dtype == MIE_F32) SCP(bf16, float);
+  else if (x_dtype == MIE_BF16 && out_dtype == MIE_BF16) SCP(bf16, bf16);
+  else MIE_FAIL("stream_copy: dtype codes x %d, out %d", x_dtype, out_dtype);
+#undef SCP
+  MIE_CHECK_LAUNCH("stream_copy");
   return 0;
 }
 

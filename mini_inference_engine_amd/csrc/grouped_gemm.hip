@@ -429,16 +429,17 @@ MIE_EXPORT int mie_grouped_glu(const void* A, int a_dtype, long lda, const void*
 // ---- router, one thread a token.  over_all == 0: the `top` largest of logits[t, :] + bias (lowest index first among
 // equals), in falling order, and the softmax over those alone.  over_all != 0: scores = softmax of logits + bias over
 // all E; chosen are the `top` largest of scores + choice_bias (same order rules); the shares are the chosen ones'
-// scores as they are (over_all == 1) or divided by their sum + 1e-20 (over_all == 2).
+// scores as they are (over_all == 1) or divided by their sum + 1e-20 (over_all == 2).  over_all 3 and 4: the same with
+// scores = sigmoid of logits + bias, every output by itself.  The shares of over_all != 0 are multiplied by `scale`.
 #define ROUTE_MAX_TOP 16
 __global__ void route_topk_kernel(const float* __restrict__ logits, long ld, const float* __restrict__ bias,
-                                  const float* __restrict__ choice_bias, int over_all, int* __restrict__ experts,
+                                  const float* __restrict__ choice_bias, int over_all, float scale, int* __restrict__ experts,
                                   float* __restrict__ shares, int T, int E, int top) {
   const int t = blockIdx.x * blockDim.x + threadIdx.x;
   if (t >= T) return;
   const float* z = logits + (size_t)t * ld;
   float largest = 0.f, total = 1.f;
-  if (over_all) {
+  if (over_all == 1 || over_all == 2) {
     largest = -INFINITY;
     for (int e = 0; e < E; ++e) largest = fmaxf(largest, z[e] + (bias ? bias[e] : 0.f));
     total = 0.f;
@@ -455,7 +456,7 @@ __global__ void route_topk_kernel(const float* __restrict__ logits, long ld, con
       if (taken) continue;
       float v = z[e] + (bias ? bias[e] : 0.f), sc = v;
       if (over_all) {
-        sc = expf(v - largest) / total;
+        sc = over_all >= 3 ? mie_sigmoid(v) : expf(v - largest) / total;
         v = sc + (choice_bias ? choice_bias[e] : 0.f);
       }
       if (best < 0 || v > bv) { best = e; bv = v; bs = sc; }
@@ -468,11 +469,13 @@ __global__ void route_topk_kernel(const float* __restrict__ logits, long ld, con
     const float first = val[0];
     for (int j = 0; j < top; ++j) { val[j] = expf(val[j] - first); sum += val[j]; }
     for (int j = 0; j < top; ++j) val[j] /= sum;
-  } else if (over_all == 2) {
+  } else if (over_all == 2 || over_all == 4) {
     float sum = 0.f;
     for (int j = 0; j < top; ++j) sum += val[j];
     for (int j = 0; j < top; ++j) val[j] /= sum + 1e-20f;
   }
+  if (over_all)
+    for (int j = 0; j < top; ++j) val[j] *= scale;
   for (int j = 0; j < top; ++j) {
     experts[(size_t)t * top + j] = chosen[j];
     shares[(size_t)t * top + j] = val[j];
@@ -485,7 +488,7 @@ __global__ void route_topk_kernel(const float* __restrict__ logits, long ld, con
 #define ROUTE_WAVE_E 128
 __global__ void __launch_bounds__(256)
 route_topk_wave_kernel(const float* __restrict__ logits, long ld, const float* __restrict__ bias,
-                       const float* __restrict__ choice_bias, int over_all, int* __restrict__ experts,
+                       const float* __restrict__ choice_bias, int over_all, float scale, int* __restrict__ experts,
                        float* __restrict__ shares, int T, int E, int top) {
   const int lane = threadIdx.x & 63, t = blockIdx.x * 4 + (threadIdx.x >> 6);
   if (t >= T) return;                        // the whole wave
@@ -497,7 +500,10 @@ route_topk_wave_kernel(const float* __restrict__ logits, long ld, const float* _
     v[i] = e < E ? z[e] + (bias ? bias[e] : 0.f) : -INFINITY;
     c[i] = e < E && over_all && choice_bias ? choice_bias[e] : 0.f;
   }
-  if (over_all) {
+  if (over_all >= 3) {
+    v[0] = lane < E ? mie_sigmoid(v[0]) : -INFINITY;
+    v[1] = lane + 64 < E ? mie_sigmoid(v[1]) : -INFINITY;
+  } else if (over_all) {
     const float largest = wave_max(fmaxf(v[0], v[1]));
     const float x0 = lane < E ? expf(v[0] - largest) : 0.f, x1 = lane + 64 < E ? expf(v[1] - largest) : 0.f;
     const float total = wave_sum(x0 + x1);
@@ -524,23 +530,24 @@ route_topk_wave_kernel(const float* __restrict__ logits, long ld, const float* _
     const float first = __shfl(mine, 0, MIE_WAVE);
     mine = lane < top ? expf(mine - first) : 0.f;
     mine /= wave_sum(mine);
-  } else if (over_all == 2) {
+  } else if (over_all == 2 || over_all == 4) {
     mine = lane < top ? mine : 0.f;
     mine /= wave_sum(mine) + 1e-20f;
   }
+  if (over_all) mine *= scale;
   if (lane < top) shares[(size_t)t * top + lane] = mine;
 }
 
-static int route_topk_launch(const float* logits, long ld, const float* bias, const float* choice_bias, int over_all,
+static int route_topk_launch(const float* logits, long ld, const float* bias, const float* choice_bias, int over_all, float scale,
                              int* experts, float* shares, int T, int E, int top, hipStream_t s) {
   if (T <= 0) return 0;
   if (E <= 0 || top <= 0 || top > E || top > ROUTE_MAX_TOP) MIE_FAIL("route_topk: top %d of %d experts (at most %d)", top, E, ROUTE_MAX_TOP);
   if (ld < E) MIE_FAIL("route_topk: row stride %ld < %d", ld, E);
   if (E <= ROUTE_WAVE_E)
-    hipLaunchKernelGGL(route_topk_wave_kernel, dim3((T + 3) / 4), dim3(256), 0, s, logits, ld, bias, choice_bias, over_all,
+    hipLaunchKernelGGL(route_topk_wave_kernel, dim3((T + 3) / 4), dim3(256), 0, s, logits, ld, bias, choice_bias, over_all, scale,
                        experts, shares, T, E, top);
   else
-    hipLaunchKernelGGL(route_topk_kernel, dim3((T + 63) / 64), dim3(64), 0, s, logits, ld, bias, choice_bias, over_all, experts,
+    hipLaunchKernelGGL(route_topk_kernel, dim3((T + 63) / 64), dim3(64), 0, s, logits, ld, bias, choice_bias, over_all, scale, experts,
                        shares, T, E, top);
   MIE_CHECK_LAUNCH("route_topk");
   return 0;
@@ -548,12 +555,13 @@ static int route_topk_launch(const float* logits, long ld, const float* bias, co
 
 MIE_EXPORT int mie_route_topk(const float* logits, long ld, const float* bias, int* experts, float* shares, int T, int E,
                               int top, hipStream_t s) {
-  return route_topk_launch(logits, ld, bias, nullptr, 0, experts, shares, T, E, top, s);
+  return route_topk_launch(logits, ld, bias, nullptr, 0, 1.f, experts, shares, T, E, top, s);
 }
 
+// sigmoid: scores are sigmoids, every output by itself, instead of a softmax over all of them
 MIE_EXPORT int mie_route_topk_all(const float* logits, long ld, const float* bias, const float* choice_bias, int* experts,
-                                  float* shares, int T, int E, int top, int renormalise, hipStream_t s) {
-  return route_topk_launch(logits, ld, bias, choice_bias, renormalise ? 2 : 1, experts, shares, T, E, top, s);
+                                  float* shares, int T, int E, int top, int renormalise, int sigmoid, float scale, hipStream_t s) {
+  return route_topk_launch(logits, ld, bias, choice_bias, (sigmoid ? 3 : 1) + (renormalise ? 1 : 0), scale, experts, shares, T, E, top, s);
 }
 
 // ---- sort the n = T * top (token, choice) pairs by expert: offs [E + 1] (where each expert's pairs start in the

@@ -38,6 +38,8 @@
 //
 // KEEP: beside the window a query sees its request's first ``keep`` keys.  The steps that hold them come before the
 // window's: place x in the order of the steps is key x up to the end of the kept steps, key x + gap behind it.
+//
+// CHUNK: the softmax over the keys of a query's own chunk of positions (the chunk size of SIG, with a softmax).
 typedef float f32x16 __attribute__((ext_vector_type(16)));
 struct __attribute__((packed, aligned(4))) Run4 { float a, b, c, d; };      // four table entries in a row, 4-byte aligned
 
@@ -81,7 +83,7 @@ __device__ __forceinline__ float pair_sum(float x) {
 // KS = 2: the waves form two halves that take the even and the odd 64-key blocks of the same queries (a step
 // brings 128 keys in, each half computes its 64) and join their results at the end: half the blocks a wave
 // for rows too short to give every SIMD two waves otherwise.
-template <int PF_WAVES, int KS, bool SIG, bool DB = false, bool KEEP = false>
+template <int PF_WAVES, int KS, bool SIG, bool DB = false, bool KEEP = false, bool CHUNK = false>
 __global__ void __launch_bounds__(PF_WAVES * 64)
 prefill_attention_kernel(const bf16* __restrict__ q, long q_stride, const bf16* __restrict__ k_cache,
                          const bf16* __restrict__ v_cache, bf16* __restrict__ out,
@@ -92,6 +94,7 @@ prefill_attention_kernel(const bf16* __restrict__ q, long q_stride, const bf16* 
                          const float* __restrict__ head_sinks) {
   static_assert(!(SIG && DB), "the distance bias is built for the softmax");
   static_assert(!(KEEP && (SIG || DB)), "kept first keys are built for the plain softmax");
+  static_assert(!(CHUNK && (SIG || DB || KEEP)), "chunks are built for the plain softmax, and for sigmoids");
   extern __shared__ __align__(16) unsigned char pf_lds[];
   constexpr int PF_THREADS = PF_WAVES * 64;
   constexpr int SUB_WAVES = PF_WAVES / KS;                   // waves of one half
@@ -175,9 +178,9 @@ prefill_attention_kernel(const bf16* __restrict__ q, long q_stride, const bf16* 
     const int kmax = p0 + end_q - 1;
     int kmin = window > 0 ? p0 + s * STRETCH - window + 1 : 0;
     kmin = kmin > 0 ? kmin : 0;
-    int q_lo = 0, tile_lo = 0;                                 // SIG: first key of the lane's query's chunk, of the tile's last query's
+    int q_lo = 0, tile_lo = 0;                                 // with chunks: first key of the lane's query's, of the tile's last query's
     float sg_c1 = 0.f, sg_c2 = 0.f, sg_c3 = 0.f;
-    if constexpr (SIG) {
+    if constexpr (SIG || CHUNK) {
       if (chunk > 0) {
         const int c_wave = tile_first / chunk * chunk, c_str = (p0 + s * STRETCH) / chunk * chunk;
         wave_kmin = wave_kmin > c_wave ? wave_kmin : c_wave;
@@ -185,6 +188,8 @@ prefill_attention_kernel(const bf16* __restrict__ q, long q_stride, const bf16* 
         q_lo = qpos / chunk * chunk;
         tile_lo = tile_last / chunk * chunk;
       }
+    }
+    if constexpr (SIG) {
       // here scale_log2 carries the plain scale
       const float hb = head_bias ? head_bias[head] : 0.f;
       const float L2E = 1.4426950408889634f;
@@ -374,7 +379,7 @@ prefill_attention_kernel(const bf16* __restrict__ q, long q_stride, const bf16* 
       }
       // every query of the tile sees every key of the block (uniform over the wave)
       const bool whole = blk + PF_BK - 1 <= tile_first &&
-                         (window <= 0 || blk >= tile_last - window + 1 || (KEEP && blk + PF_BK <= keep)) && (!SIG || blk >= tile_lo);
+                         (window <= 0 || blk >= tile_last - window + 1 || (KEEP && blk + PF_BK <= keep)) && (!(SIG || CHUNK) || blk >= tile_lo);
       if constexpr (DB) {
 #pragma unroll
         for (int u = 0; u < 2; ++u)
@@ -440,7 +445,8 @@ prefill_attention_kernel(const bf16* __restrict__ q, long q_stride, const bf16* 
           for (int i = 0; i < 16; ++i) S[u][i] = fast_exp2(fmaf(S[u][i], sl2, -m_new));
       } else {
         const int hi = tile_ok ? qpos : -1;                    // a tile that does not exist sees nothing
-        const int lo = window > 0 ? hi - window + 1 : 0;
+        int lo = window > 0 ? hi - window + 1 : 0;
+        if constexpr (CHUNK) lo = lo > q_lo ? lo : q_lo;
         float mx = -INFINITY;
 #pragma unroll
         for (int u = 0; u < 2; ++u)
@@ -643,9 +649,11 @@ static int prefill_attention_launch(const void* q, long q_stride, const void* k_
   if (grid.y > 65535 || grid.z > 65535) MIE_FAIL("prefill_attention: grid too large (%d rows)", rows);
   const float scale_log2 = sigmoid ? scale : scale * 1.4426950408889634f;      // the sigmoid kernels fold their own constants
   // more LDS than a kernel gets by default is asked for once per kernel and device
-  static bool lds_allowed[12][64] = {};
+  const bool chunked = chunk > 0 && !sigmoid;
+  if (chunked && (keep > 0 || dist_bias)) MIE_FAIL("prefill_attention: chunks beside kept keys or a distance bias are not built");
+  static bool lds_allowed[15][64] = {};
   auto launch = [&](auto kernel, int waves, int lds_bytes) -> int {
-    const int which = kind + (sigmoid ? 3 : 0) + (dist_bias ? 6 : 0) + (keep > 0 ? 9 : 0);
+    const int which = kind + (sigmoid ? 3 : 0) + (dist_bias ? 6 : 0) + (keep > 0 ? 9 : 0) + (chunked ? 12 : 0);
     if (lds_bytes > 64 * 1024 && !lds_allowed[which][dev]) {
       hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, lds_bytes);
       if (e != hipSuccess) MIE_FAIL("prefill_attention: %d bytes of LDS refused: %s", lds_bytes, hipGetErrorString(e));
@@ -658,18 +666,21 @@ static int prefill_attention_launch(const void* q, long q_stride, const void* k_
     return 0;
   };
   int rc = 0;
-  const bool plain = !sigmoid && !dist_bias && keep == 0;
+  const bool plain = !sigmoid && !dist_bias && keep == 0 && !chunked;
   if constexpr (PF_MAX_WAVES == 8) {
     if (kind == EIGHT_QUERIES && dist_bias) rc = launch(prefill_attention_kernel<8, 1, false, true>, 8, 2 * PF_BUF);
     if (kind == EIGHT_KEYS && dist_bias) rc = launch(prefill_attention_kernel<8, 2, false, true>, 8, 4 * PF_BUF);
     if (kind == EIGHT_QUERIES && plain) rc = launch(prefill_attention_kernel<8, 1, false>, 8, 2 * PF_BUF);
     if (kind == EIGHT_KEYS && plain) rc = launch(prefill_attention_kernel<8, 2, false>, 8, 4 * PF_BUF);
+    if (kind == EIGHT_QUERIES && chunked) rc = launch(prefill_attention_kernel<8, 1, false, false, false, true>, 8, 2 * PF_BUF);
+    if (kind == EIGHT_KEYS && chunked) rc = launch(prefill_attention_kernel<8, 2, false, false, false, true>, 8, 4 * PF_BUF);
     if (kind == EIGHT_QUERIES && keep > 0) rc = launch(prefill_attention_kernel<8, 1, false, false, true>, 8, 2 * PF_BUF);
     if (kind == EIGHT_KEYS && keep > 0) rc = launch(prefill_attention_kernel<8, 2, false, false, true>, 8, 4 * PF_BUF);
     if (kind == EIGHT_QUERIES && sigmoid) rc = launch(prefill_attention_kernel<8, 1, true>, 8, 2 * PF_BUF);
     if (kind == EIGHT_KEYS && sigmoid) rc = launch(prefill_attention_kernel<8, 2, true>, 8, 4 * PF_BUF);
   }
   if (kind == FOUR && dist_bias) rc = launch(prefill_attention_kernel<4, 1, false, true>, 4, 2 * PF_BUF);
+  if (kind == FOUR && chunked) rc = launch(prefill_attention_kernel<4, 1, false, false, false, true>, 4, 2 * PF_BUF);
   if (kind == FOUR && keep > 0) rc = launch(prefill_attention_kernel<4, 1, false, false, true>, 4, 2 * PF_BUF);
   if (kind == FOUR && plain) rc = launch(prefill_attention_kernel<4, 1, false>, 4, 2 * PF_BUF);
   if (kind == FOUR && sigmoid) rc = launch(prefill_attention_kernel<4, 1, true>, 4, 2 * PF_BUF);
@@ -733,4 +744,17 @@ MIE_EXPORT int mie_prefill_attention_kept(const void* q, long q_stride, const vo
   return prefill_attention_launch(q, q_stride, k_cache, v_cache, out, block_tables, max_blocks, row_start, row_position,
                                   first_row, rows, max_row_tokens, Hq, Hkv, head_dim, page, scale, window, -INFINITY, stream,
                                   false, 0, 0.f, nullptr, nullptr, 0, keep, head_sinks);
+}
+
+// The softmax over the keys of a query's own chunk of positions, from floor(position / chunk) chunk on (and over the last
+// ``window`` of them, if that is not 0).
+MIE_EXPORT int mie_prefill_attention_chunked(const void* q, long q_stride, const void* k_cache, const void* v_cache, void* out,
+                                             const int* block_tables, int max_blocks, const int* row_start,
+                                             const int* row_position, int first_row, int rows, int max_row_tokens, int Hq,
+                                             int Hkv, int head_dim, int page, float scale, int window, int chunk,
+                                             hipStream_t stream) {
+  if (chunk < 1) MIE_FAIL("prefill_attention_chunked: chunks of %d positions", chunk);
+  return prefill_attention_launch(q, q_stride, k_cache, v_cache, out, block_tables, max_blocks, row_start, row_position,
+                                  first_row, rows, max_row_tokens, Hq, Hkv, head_dim, page, scale, window, -INFINITY, stream,
+                                  false, chunk);
 }

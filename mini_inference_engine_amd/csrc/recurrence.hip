@@ -151,17 +151,18 @@ short_conv_tile_kernel(const float* __restrict__ x, long ldx, const float* __res
   }
 }
 
-// the row's last K - 1 inputs (old tail, then this step's x), oldest first, into tail[slot]; a thread a (row, channel)
+// the row's last K - 1 inputs (old tail, then this step's x (+ in_bias)), oldest first, into tail[slot]; a thread a (row, channel)
 __global__ void __launch_bounds__(256)
-conv_tail_move_kernel(const float* __restrict__ x, long ldx, float* __restrict__ tail, const int* __restrict__ row_start,
-                      const int* __restrict__ slots, int C, int K) {
+conv_tail_move_kernel(const float* __restrict__ x, long ldx, const float* __restrict__ in_bias, float* __restrict__ tail,
+                      const int* __restrict__ row_start, const int* __restrict__ slots, int C, int K) {
   const int r = blockIdx.x, c = blockIdx.y * blockDim.x + threadIdx.x;
   if (c >= C) return;
   const int a0 = row_start[r], n = row_start[r + 1] - a0, keep = K - 1;
+  const float b = in_bias ? in_bias[c] : 0.f;
   float* tl = tail + (size_t)slots[r] * keep * C;
   for (int i = 0; i < keep; ++i) {
     const int src = n + i;                     // place in the joined sequence of keep + n inputs
-    tl[(size_t)i * C + c] = src < keep ? tl[(size_t)src * C + c] : x[(size_t)(a0 + src - keep) * ldx + c];
+    tl[(size_t)i * C + c] = src < keep ? tl[(size_t)src * C + c] : x[(size_t)(a0 + src - keep) * ldx + c] + b;
   }
 }
 
@@ -391,11 +392,11 @@ MIE_EXPORT int mie_short_conv(const float* x, long ldx, const float* taps, const
   return 0;
 }
 
-MIE_EXPORT int mie_conv_tail_move(const float* x, long ldx, float* tail, const int* row_start, const int* slots, int rows, int C,
-                                  int K, hipStream_t s) {
+MIE_EXPORT int mie_conv_tail_move(const float* x, long ldx, const float* in_bias, float* tail, const int* row_start, const int* slots,
+                                  int rows, int C, int K, hipStream_t s) {
   if (rows <= 0 || K <= 1) return 0;
   if (C <= 0 || ldx < C || !x || !tail || !row_start || !slots) MIE_FAIL("conv_tail_move: %d channels, row stride %ld", C, ldx);
-  hipLaunchKernelGGL(conv_tail_move_kernel, dim3(rows, (C + 255) / 256), dim3(256), 0, s, x, ldx, tail, row_start, slots, C, K);
+  hipLaunchKernelGGL(conv_tail_move_kernel, dim3(rows, (C + 255) / 256), dim3(256), 0, s, x, ldx, in_bias, tail, row_start, slots, C, K);
   MIE_CHECK_LAUNCH("conv_tail_move");
   return 0;
 }

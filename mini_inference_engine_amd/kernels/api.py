@@ -53,22 +53,36 @@ class Normed:
 
 
 class NormedLayer(Normed):
-    """The same for a layer norm with weight and bias: layernorm(residual (+ pending)) * weight + bias."""
+    """The same for a layer norm with weight and bias (or without: None): layernorm(residual (+ pending)) * weight + bias.
+    ``pending_bias``: a vector that is still to be added to every row of the stream too (BiasedBranch)."""
 
-    def __init__(self, ops, pending, residual, weight, bias, eps, rows=None):
+    def __init__(self, ops, pending, residual, weight, bias, eps, rows=None, pending_bias=None):
         super().__init__(ops, pending, residual, weight, eps, rows)
-        self.bias = bias
+        self.bias, self.pending_bias = bias, pending_bias
 
     def with_rows(self, rows):
-        return NormedLayer(self.ops, self.pending, self.residual, self.weight, self.bias, self.eps, rows)
+        return NormedLayer(self.ops, self.pending, self.residual, self.weight, self.bias, self.eps, rows, self.pending_bias)
 
     def materialize(self, out_dtype=None):
         if self._value is None:
+            more = {} if self.pending_bias is None else {"x_bias": self.pending_bias}
             self._value = self.ops.add_layernorm(self.pending, self.residual, self.weight, self.bias, self.eps,
-                                                 out_dtype=out_dtype, rows=self.rows)
+                                                 out_dtype=out_dtype, rows=self.rows, **more)
             if self.rows is None:
-                self.pending = None
+                self.pending = self.pending_bias = None
         return self._value
+
+
+class BiasedBranch:
+    """A branch output that is still to be added to the stream together with a vector of its own: stream += value + bias, bias
+    float32 [width] for every row.  ``value`` None: the output itself is in the stream already, the vector is not.  A layer
+    norm adds both on its way (NormedLayer); ``float()`` is what anyone else has to add."""
+
+    def __init__(self, value, bias):
+        self.value, self.bias = value, bias
+
+    def float(self):
+        return self.bias if self.value is None else self.value.float() + self.bias
 
 
 class NormedBranch:
@@ -109,10 +123,16 @@ class KernelBackend:
         """Row counts of steps that will recur (the batch sizes decode graphs are captured at, the token budget
         of a step): a backend may spend time once, outside any capture, to choose its kernels for them."""
 
-    def embedding(self, ids, table, taken_from=None, earlier_tokens=None, scale=1.0):
+    def embedding(self, ids, table, taken_from=None, earlier_tokens=None, scale=1.0, copy=None):
         """stream[t, :] = float(table[ids[t], :]) * scale -> [T, width] float32.  With ``taken_from`` (int32 [T]):
         where it is >= 0 the token is ``earlier_tokens[taken_from[t]]`` instead of ``ids[t]`` (a token the
-        step before chose, read on the device because the host has not seen it yet)."""
+        step before chose, read on the device because the host has not seen it yet).  ``copy`` ([T, width] in the
+        activation dtype, rows may be further apart) receives the rows too, rounded once."""
+        raise NotImplementedError
+
+    def stream_copy(self, x, stream, out, x_bias=None):
+        """out = stream (+ float(x)) (+ x_bias) in the activation dtype, rounded once; ``out`` [T, width] (rows may be further
+        apart), x of any float dtype, x_bias float32 [width].  The float32 stream itself is left as it is."""
         raise NotImplementedError
 
     def add_rmsnorm(self, x, residual, weight, eps, out_dtype=None, rows=None):
@@ -158,15 +178,15 @@ class KernelBackend:
         """t = cap * tanh(t * scale / cap) in place (float32; ``cap`` None: t * scale), returns t."""
         raise NotImplementedError
 
-    def add_layernorm(self, x, residual, weight, bias, eps, out_dtype=None, rows=None):
-        """If ``x`` is given: residual += float(x), in place.  y = (residual - mean) / sqrt(var + eps) * weight + bias,
-        mean and var (the mean of the squared deviations) of each row, all in float32 (weight, bias float32 [width]),
-        rounded once to ``out_dtype`` (default act_dtype).  With ``rows`` only those rows are computed, y is
+    def add_layernorm(self, x, residual, weight, bias, eps, out_dtype=None, rows=None, x_bias=None):
+        """If ``x`` is given: residual += float(x), in place; likewise ``x_bias`` (float32 [width]) to every row.  y = (residual - mean) / sqrt(var + eps) * weight + bias,
+        mean and var (the mean of the squared deviations) of each row, all in float32 (weight, bias float32 [width]; bias may be
+        None), rounded once to ``out_dtype`` (default act_dtype).  With ``rows`` only those rows are computed, y is
         [len(rows), width] and residual is not modified."""
         raise NotImplementedError
 
     def branch_layernorm_add(self, y, stream, weight, bias, eps, next_norm=None):
-        """stream += layernorm(y) * weight + bias, row by row in float32 (y [T, width] of any float dtype).  With
+        """stream += layernorm(y) * weight + bias (None: no bias), row by row in float32 (y [T, width] of any float dtype).  With
         ``next_norm`` = (weight, bias, eps) also returns that layer norm of the updated stream in the activation dtype
         (a backend may do both in one kernel); else None."""
         raise NotImplementedError
@@ -229,12 +249,13 @@ class KernelBackend:
         raise NotImplementedError
 
     # ---- routed experts
-    def route_topk(self, logits, bias, top, over="chosen", choice_bias=None, renormalise=False):
+    def route_topk(self, logits, bias, top, over="chosen", choice_bias=None, renormalise=False, scale=1.0):
         """logits [T, E] float32 (+ bias [E]).  ``over`` "chosen": the ``top`` largest of a token (lowest index first
         among equals), in falling order, and the softmax over those alone.  ``over`` "all": scores = softmax over all
         E; chosen are the ``top`` largest of scores + choice_bias (float32 [E] or None; lowest index first among
         equals, falling order) and the shares are the chosen ones' scores as they are, or, with ``renormalise``,
-        divided by their sum + 1e-20.
+        divided by their sum + 1e-20.  ``over`` "sigmoid": the same with scores = sigmoid of every output by itself.
+        ``scale``: factor on the shares ("all" and "sigmoid").
         -> (experts [T, top] int32, shares [T, top] float32)."""
         raise NotImplementedError
 
@@ -282,7 +303,7 @@ class KernelBackend:
     def qkv_finish(self, sums, q_col, k_col, v_col, num_q_heads, num_kv_heads, dim, vdim, padded_dim, positions, inv_freq,
                    layout, k_cache, v_cache, slot_mapping, q_norm=None, k_norm=None, eps=0.0, q_head_scale=None,
                    norm_per_head=False, col_bias=None, position_temperature=None, rotation_scale=1.0, conv=None,
-                   values_out=None, value_mix=None):
+                   values_out=None, value_mix=None, norm_turned=False):
         """What lies between a q/k/v projection's float32 sums [T, *] and attention, in 32-bit: queries are columns
         [q_col, q_col + Hq dim), keys [k_col, k_col + Hkv dim), values [v_col, v_col + Hkv vdim), or, with ``v_col``
         None, the keys as projected (vdim = dim).  ``col_bias`` (float32, one number a column of the sums): the
@@ -298,7 +319,9 @@ class KernelBackend:
         ``conv`` = (taps, tail, step): before anything else every channel c of the three projections, which then lie side by
         side from q_col on (C = (Hq + Hkv) dim + Hkv vdim of them), passes y_t = sum_j taps[c, j] u_(t - K + 1 + j) (taps float32
         [C, K]) over its row's tokens; inputs before the row's first token come from ``tail`` [slots, max(1, K - 1), C] float32,
-        which moves on (as in ``residual_conv``).  ``rotation_scale``: factor on every cosine and sine.  ``values_out`` (float32
+        which moves on (as in ``residual_conv``); ``col_bias`` is added before the convolution (the tail holds biased inputs, and
+        zeros at a request's start).  ``norm_turned``: after the rotation every query and key head is divided by its root mean
+        square over dim (with eps inside; no weights).  ``rotation_scale``: factor on every cosine and sine.  ``values_out`` (float32
         [T, Hkv vdim]) receives the values; ``value_mix`` = (lam, other float32 [T, Hkv vdim]): what is cached as values is
         (1 - lam) v + lam other.
         -> q [T, Hq * P] in the activation dtype, zeros beyond dim."""
@@ -352,6 +375,19 @@ class KernelBackend:
         [slots, H, dim, dim] float32 (S[i, j]: key channel i, value channel j), left there afterwards:
         S <- diag(decay) S - (a * u) (u^T S) + k v^T with both terms of the old S; o = S^T r.
         -> rmsnorm(o over a head, eps) * norm_weight * sigmoid(g)  [T, H * dim] in the activation dtype."""
+        raise NotImplementedError
+
+    def gated_delta(self, u, q_col, k_col, v_col, sums, beta_col, decay_col, gate_col, num_heads, num_kv_heads, dim, vdim,
+                    w_decay, rate, decay_bias, w_gate, q_scale, norm_weight, eps, state, step):
+        """A gated delta rule with a decay per key channel.  u float32 [T, *]: queries and keys from q_col, k_col on (kv_heads
+        dim each; head h reads h // (heads / kv_heads)), values from v_col on (heads vdim); sums float32 [T, *]: beta from beta_col
+        on (one a head), the inner activations of decays and gate from decay_col, gate_col on (w_decay.shape[1] and
+        w_gate.shape[1] of them).  In 32-bit: q, k over sqrt(sum of squares + 1e-6) head by head, q times q_scale;
+        g = exp(-rate softplus(w_decay a + decay_bias)) (w_decay [heads dim, *], rate [heads]); beta <- sigmoid(beta).  Per row
+        and head, tokens in order, from the row's slot of ``state`` [slots, heads, dim, vdim], left there afterwards:
+        S <- diag(g) S;  w = beta (v - S^T k);  S <- S + k w^T;  o = S^T q.
+        -> rmsnorm(o over a head, eps) * norm_weight [vdim] * sigmoid(w_gate b)  [T, heads vdim] in the activation dtype
+        (b the gate's inner activations, w_gate [heads vdim, *])."""
         raise NotImplementedError
 
     def normed_sum_add(self, stream, ys, weights, eps, scale):

@@ -147,8 +147,8 @@ class HipBackend(KernelBackend):
         return out
 
     # ----------------------------------------------------------------- ops
-    def embedding(self, ids, table, taken_from=None, earlier_tokens=None, scale=1.0):
-        self._on_device(ids, table, taken_from, earlier_tokens)
+    def embedding(self, ids, table, taken_from=None, earlier_tokens=None, scale=1.0, copy=None):
+        self._on_device(ids, table, taken_from, earlier_tokens, copy)
         if ids.dtype != torch.int32 or ids.dim() != 1 or not ids.is_contiguous():
             raise ValueError("embedding: ids must be contiguous int32 [T]")
         if taken_from is not None:
@@ -158,10 +158,30 @@ class HipBackend(KernelBackend):
         if table.dim() != 2 or not table.is_contiguous():
             raise ValueError("embedding: table must be contiguous [vocab, width]")
         T, (V, W) = ids.shape[0], table.shape
+        if copy is not None and (tuple(copy.shape) != (T, W) or copy.stride(1) != 1):
+            raise ValueError(f"embedding: copy {tuple(copy.shape)}, expected {(T, W)} with unit inner stride")
         out = torch.empty((T, W), dtype=torch.float32, device=table.device)
         lib = self.lib("embed_norm")
         library.check(lib, lib.mie_embedding(_ptr(ids), _ptr(table), _code(table.dtype), _ptr(out), T, W, V,
-                                             _ptr(taken_from), _ptr(earlier_tokens), float(scale), self._stream()))
+                                             _ptr(taken_from), _ptr(earlier_tokens), float(scale), _ptr(copy),
+                                             F32 if copy is None else _code(copy.dtype), 0 if copy is None else copy.stride(0),
+                                             self._stream()))
+        return out
+
+    def stream_copy(self, x, stream, out, x_bias=None):
+        self._on_device(x, stream, out, x_bias)
+        if stream.dtype != torch.float32 or stream.dim() != 2 or not stream.is_contiguous():
+            raise ValueError("stream_copy: the stream must be contiguous float32 [T, width]")
+        T, W = stream.shape
+        if x is not None and (tuple(x.shape) != (T, W) or not x.is_contiguous()):
+            raise ValueError(f"stream_copy: x {tuple(x.shape)} does not match the stream {(T, W)}")
+        if tuple(out.shape) != (T, W) or out.stride(1) != 1:
+            raise ValueError(f"stream_copy: out {tuple(out.shape)}, expected {(T, W)} with unit inner stride")
+        if x_bias is not None:
+            self._f32_vector(x_bias, W, "stream_copy: x_bias")
+        lib = self.lib("embed_norm")
+        library.check(lib, lib.mie_stream_copy(_ptr(x), F32 if x is None else _code(x.dtype), _ptr(x_bias), _ptr(stream), _ptr(out),
+                                               _code(out.dtype), out.stride(0), T, W, self._stream()))
         return out
 
     def add_rmsnorm(self, x, residual, weight, eps, out_dtype=None, rows=None):
@@ -473,8 +493,8 @@ class HipBackend(KernelBackend):
         library.check(lib, lib.mie_scale_softcap(_ptr(t), t.numel(), float(scale), float(cap or 0.0), self._stream()))
         return t
 
-    def add_layernorm(self, x, residual, weight, bias, eps, out_dtype=None, rows=None):
-        self._on_device(x, residual, weight, bias, rows)
+    def add_layernorm(self, x, residual, weight, bias, eps, out_dtype=None, rows=None, x_bias=None):
+        self._on_device(x, residual, weight, bias, rows, x_bias)
         out_dtype = out_dtype or self.act_dtype
         if residual.dtype != torch.float32 or residual.dim() != 2 or not residual.is_contiguous():
             raise ValueError("add_layernorm: the residual stream must be contiguous float32 [T, width]")
@@ -482,7 +502,9 @@ class HipBackend(KernelBackend):
         if x is not None and (tuple(x.shape) != (T, W) or not x.is_contiguous()):
             raise ValueError(f"add_layernorm: x {tuple(x.shape)} does not match the stream {(T, W)}")
         self._f32_vector(weight, W, "add_layernorm: weight")
-        self._f32_vector(bias, W, "add_layernorm: bias")
+        for name, t in (("bias", bias), ("x_bias", x_bias)):
+            if t is not None:
+                self._f32_vector(t, W, f"add_layernorm: {name}")
         n = T
         if rows is not None:
             if rows.dtype != torch.int32 or rows.dim() != 1 or not rows.is_contiguous():
@@ -490,8 +512,8 @@ class HipBackend(KernelBackend):
             n = rows.shape[0]
         y = torch.empty((n, W), dtype=out_dtype, device=residual.device)
         lib = self.lib("layer_norm")
-        library.check(lib, lib.mie_add_layernorm(_ptr(x), _code(x.dtype) if x is not None else F32, _ptr(residual), _ptr(weight),
-                                                 _ptr(bias), _ptr(y), _code(out_dtype), _ptr(rows), n, W, float(eps),
+        library.check(lib, lib.mie_add_layernorm(_ptr(x), _code(x.dtype) if x is not None else F32, _ptr(x_bias), _ptr(residual),
+                                                 _ptr(weight), _ptr(bias), _ptr(y), _code(out_dtype), _ptr(rows), n, W, float(eps),
                                                  self._stream()))
         return y
 
@@ -503,13 +525,15 @@ class HipBackend(KernelBackend):
         if tuple(y.shape) != (T, W) or not y.is_contiguous():
             raise ValueError(f"branch_layernorm_add: y {tuple(y.shape)} does not match the stream {(T, W)}")
         self._f32_vector(weight, W, "branch_layernorm_add: weight")
-        self._f32_vector(bias, W, "branch_layernorm_add: bias")
+        if bias is not None:
+            self._f32_vector(bias, W, "branch_layernorm_add: bias")
         x, nw, nb, ne = None, None, None, 0.0
         if next_norm is not None:
             nw, nb, ne = next_norm
             self._on_device(nw, nb)
             self._f32_vector(nw, W, "branch_layernorm_add: the next norm's weight")
-            self._f32_vector(nb, W, "branch_layernorm_add: the next norm's bias")
+            if nb is not None:
+                self._f32_vector(nb, W, "branch_layernorm_add: the next norm's bias")
             x = torch.empty((T, W), dtype=self.act_dtype, device=stream.device)
         lib = self.lib("layer_norm")
         library.check(lib, lib.mie_branch_layernorm_add(_ptr(y), _code(y.dtype), _ptr(stream), _ptr(weight), _ptr(bias), float(eps),
@@ -740,10 +764,11 @@ class HipBackend(KernelBackend):
         return out
 
     # ---- routed experts
-    def route_topk(self, logits, bias, top, over="chosen", choice_bias=None, renormalise=False):
+    def route_topk(self, logits, bias, top, over="chosen", choice_bias=None, renormalise=False, scale=1.0):
         self._on_device(logits, bias, choice_bias)
-        if over not in ("chosen", "all") or ((choice_bias is not None or renormalise) and over != "all"):
-            raise ValueError(f"route_topk: shares over {over!r} (chosen or all; a choice bias or renormalised shares go with all)")
+        if over not in ("chosen", "all", "sigmoid") or ((choice_bias is not None or renormalise or scale != 1.0) and over == "chosen"):
+            raise ValueError(f"route_topk: shares over {over!r} (chosen, all or sigmoid; a choice bias, renormalised shares and a "
+                             "factor on them go with the latter two)")
         if logits.dtype != torch.float32 or logits.dim() != 2 or logits.stride(1) != 1:
             raise ValueError("route_topk: logits must be float32 [T, experts] with unit inner stride")
         T, E = logits.shape
@@ -754,11 +779,12 @@ class HipBackend(KernelBackend):
         experts = torch.empty((T, top), dtype=torch.int32, device=logits.device)
         shares = torch.empty((T, top), dtype=torch.float32, device=logits.device)
         lib = self.lib("grouped_gemm")
-        if over == "all":
+        if over != "chosen":
             if choice_bias is not None:
                 self._f32_vector(choice_bias, E, "route_topk: choice bias")
             library.check(lib, lib.mie_route_topk_all(_ptr(logits), logits.stride(0), _ptr(bias), _ptr(choice_bias), _ptr(experts),
-                                                      _ptr(shares), T, E, top, int(bool(renormalise)), self._stream()))
+                                                      _ptr(shares), T, E, top, int(bool(renormalise)), int(over == "sigmoid"), float(scale),
+                                                      self._stream()))
             return experts, shares
         library.check(lib, lib.mie_route_topk(_ptr(logits), logits.stride(0), _ptr(bias), _ptr(experts), _ptr(shares), T, E, top,
                                               self._stream()))
@@ -929,7 +955,7 @@ class HipBackend(KernelBackend):
     def qkv_finish(self, sums, q_col, k_col, v_col, num_q_heads, num_kv_heads, dim, vdim, padded_dim, positions, inv_freq,
                    layout, k_cache, v_cache, slot_mapping, q_norm=None, k_norm=None, eps=0.0, q_head_scale=None,
                    norm_per_head=False, col_bias=None, position_temperature=None, rotation_scale=1.0, conv=None,
-                   values_out=None, value_mix=None):
+                   values_out=None, value_mix=None, norm_turned=False):
         self._on_device(sums, positions, inv_freq, k_cache, v_cache, slot_mapping, q_norm, k_norm, q_head_scale, col_bias)
         coef, every = 0.0, 0
         if position_temperature is not None:
@@ -967,10 +993,12 @@ class HipBackend(KernelBackend):
         # rows 64 bytes apart from a multiple of their length, as the attention kernels like their q rows
         q = torch.empty((T, Hq * P), dtype=self.act_dtype, device=sums.device)
         lib = self.lib("attention_prep")
-        if conv is not None or rotation_scale != 1.0 or values_out is not None or value_mix is not None:
+        if norm_turned and (q_norm is not None or k_norm is not None):
+            raise ValueError("qkv_finish: norms after the rotation have no weights")
+        if conv is not None or rotation_scale != 1.0 or values_out is not None or value_mix is not None or norm_turned:
             return self._qkv_conv_finish(q, sums, q_col, k_col, v_col, Hq, Hkv, dim, vdim, P, page, positions, inv_freq, nf, layout,
                                          k_cache, v_cache, slot_mapping, q_norm, k_norm, eps, rotation_scale, conv, values_out, value_mix,
-                                         plain=q_head_scale is None and col_bias is None and position_temperature is None
+                                         col_bias, norm_turned, plain=q_head_scale is None and position_temperature is None
                                          and (norm_per_head or (q_norm is None and k_norm is None)))
         library.check(lib, lib.mie_qkv_finish(
             _ptr(sums), sums.stride(0), q_col, k_col, -1 if v_col is None else v_col, _ptr(q_norm), _ptr(k_norm), float(eps),
@@ -980,13 +1008,14 @@ class HipBackend(KernelBackend):
         return q
 
     def _qkv_conv_finish(self, q, sums, q_col, k_col, v_col, Hq, Hkv, dim, vdim, P, page, positions, inv_freq, nf, layout, k_cache,
-                         v_cache, slot_mapping, q_norm, k_norm, eps, rotation_scale, conv, values_out, value_mix, plain):
+                         v_cache, slot_mapping, q_norm, k_norm, eps, rotation_scale, conv, values_out, value_mix, col_bias, norm_turned,
+                         plain):
         """The part of ``qkv_finish`` that convolves the projections, scales the rotation or shares values (operands checked)
         -> q."""
         T, dev = sums.shape[0], sums.device
-        if not plain or layout != "half" or conv is None:
-            raise ValueError("qkv_finish: a scaled rotation and shared values are built for convolved projections whose halves turn, "
-                             "with norms head by head and without biases and temperatures")
+        if not plain or conv is None:
+            raise ValueError("qkv_finish: a scaled rotation, norms after it and shared values are built for convolved projections, with "
+                             "norms head by head and without temperatures")
         taps, tail, step = conv
         self._on_device(taps, tail, values_out)
         C = (Hq + Hkv) * dim + Hkv * vdim
@@ -1007,12 +1036,13 @@ class HipBackend(KernelBackend):
         single = step.num_rows == T
         lib = self.lib("attention_prep")
         library.check(lib, lib.mie_qkv_conv_finish(
-            _ptr(sums), sums.stride(0), q_col, _ptr(taps), _ptr(tail), _ptr(step.token_row), _ptr(step.row_start), _ptr(step.state_slots),
-            K, int(single), _ptr(q_norm), _ptr(k_norm), float(eps), _ptr(inv_freq), nf, float(rotation_scale), _ptr(positions),
+            _ptr(sums), sums.stride(0), q_col, c_void_p(0 if col_bias is None else col_bias.data_ptr() + 4 * q_col), _ptr(taps), _ptr(tail),
+            _ptr(step.token_row), _ptr(step.row_start), _ptr(step.state_slots), K, int(single), _ptr(q_norm), _ptr(k_norm), float(eps),
+            int(bool(norm_turned)), _ptr(inv_freq), nf, self.LAYOUTS[layout], float(rotation_scale), _ptr(positions),
             _ptr(slot_mapping), _ptr(values_out), _ptr(other), mix, _ptr(q), _ptr(k_cache), _ptr(v_cache), _code(self.act_dtype), T, Hq,
             Hkv, dim, vdim, P, page, self._stream()))
         if not single:
-            self._move_tail(sums, q_col, C, K, tail, step)
+            self._move_tail(sums, q_col, C, K, tail, step, col_bias)
         return q
 
     def _check_tail(self, what, tail, C, K, step, T):
@@ -1022,10 +1052,11 @@ class HipBackend(KernelBackend):
         if int(step.host["state_slots"].max()) >= tail.shape[0]:
             raise ValueError(f"{what}: a state slot beyond the tail's slots")
 
-    def _move_tail(self, x, col, C, K, tail, step):
-        """The rows' last K - 1 inputs (columns [col, col + C) of x, operands checked) into their slots of ``tail``."""
+    def _move_tail(self, x, col, C, K, tail, step, col_bias=None):
+        """The rows' last K - 1 inputs (columns [col, col + C) of x (+ col_bias), operands checked) into their slots of ``tail``."""
         lib = self.lib("recurrence")
-        library.check(lib, lib.mie_conv_tail_move(c_void_p(x.data_ptr() + 4 * col), x.stride(0), _ptr(tail), _ptr(step.row_start),
+        library.check(lib, lib.mie_conv_tail_move(c_void_p(x.data_ptr() + 4 * col), x.stride(0),
+                                                  c_void_p(0 if col_bias is None else col_bias.data_ptr() + 4 * col), _ptr(tail), _ptr(step.row_start),
                                                   _ptr(step.state_slots), step.num_rows, C, K, self._stream()))
 
     def gate_heads(self, o, gate, gate_col, num_heads, vdim, padded_dim, out=None, scale=1.0):
@@ -1195,6 +1226,46 @@ class HipBackend(KernelBackend):
             _ptr(decay_bias), float(decay_scale), _ptr(removal_bias), _ptr(norm_weight), float(eps), _ptr(state),
             _ptr(step.row_start), _ptr(step.state_slots), _ptr(prep), _ptr(out), _code(out.dtype), T, step.num_rows, H, d,
             chunk, chunks, _ptr(summaries), _ptr(starts), self._stream()))
+        return out
+
+    GATED_DELTA_CHUNKED_MAX_DIM = 128     # wider keys always run token by token (a chunk's keys, queries and decays share the LDS)
+
+    def gated_delta(self, u, q_col, k_col, v_col, sums, beta_col, decay_col, gate_col, num_heads, num_kv_heads, dim, vdim,
+                    w_decay, rate, decay_bias, w_gate, q_scale, norm_weight, eps, state, step):
+        self._on_device(u, sums, w_decay, rate, decay_bias, w_gate, norm_weight, state)
+        H, G, d, dv, T = num_heads, num_kv_heads, dim, vdim, u.shape[0]
+        if G < 1 or H % G or sums.shape[0] != T or u.stride(1) != 1:
+            raise ValueError(f"gated_delta: {H} heads on {G} query/key heads, {T} and {sums.shape[0]} tokens")
+        for name, col, n in (("queries", q_col, G * d), ("keys", k_col, G * d), ("values", v_col, H * dv)):
+            self._f32_columns(u, col, n, f"gated_delta: {name}")
+        for name, col, w, n in (("decays", decay_col, w_decay, H * d), ("gate", gate_col, w_gate, H * dv)):
+            if w.dim() != 2 or w.shape[0] != n or w.shape[1] % 16 or col % 16:
+                raise ValueError(f"gated_delta: {name}: matrix {tuple(w.shape)} for {n} channels, column {col} (inner sizes and columns in 16s)")
+            self._f32_vector(w, w.numel(), f"gated_delta: {name}")
+            self._f32_columns(sums, col, w.shape[1], f"gated_delta: {name}")
+        self._f32_columns(sums, beta_col, H, "gated_delta: beta")
+        for name, t, n in (("rate", rate, H), ("decay_bias", decay_bias, H * d), ("norm_weight", norm_weight, dv)):
+            self._f32_vector(t, n, f"gated_delta: {name}")
+        self._check_state("gated_delta", state, (H, d, dv), step, T)
+        out = torch.empty((T, H * dv), dtype=self.act_dtype, device=u.device)
+        la = torch.empty((T, H * d), dtype=torch.float32, device=u.device)
+        gate = torch.empty((T, H * dv), dtype=torch.float32, device=u.device)
+        lib = self.lib("gated_delta")
+        longest = int(getattr(step, "max_row_tokens", 0) or (step.host["row_start"][1:] - step.host["row_start"][:-1]).max())
+        whole, chunks, dp, vp, scratch = step.num_rows, 0, 0, 0, None
+        if longest > self.STATE_CHUNK and not self.true_fp32 and d <= self.GATED_DELTA_CHUNKED_MAX_DIM:
+            # rows of many tokens: chunks side by side, single-token rows (they lead the batch) token by token.  Whether a portion
+            # takes this path depends on the step's longest row alone; the two paths differ by rounding, so the 32-bit mode
+            # keeps to one.
+            whole, chunks = step.num_decode_rows, -(-longest // self.STATE_CHUNK)
+            dp, vp = (max(32, 1 << (n - 1).bit_length()) for n in (d, dv))
+            units = (step.num_rows - whole) * chunks * H
+            scratch = torch.empty(units * lib.mie_gated_delta_unit_floats(dp, vp), dtype=torch.float32, device=u.device)
+        library.check(lib, lib.mie_gated_delta(
+            _ptr(u), u.stride(0), q_col, k_col, v_col, _ptr(sums), sums.stride(0), beta_col, decay_col, gate_col, _ptr(w_decay), w_decay.shape[1],
+            _ptr(rate), _ptr(decay_bias), _ptr(w_gate), w_gate.shape[1], float(q_scale), _ptr(norm_weight), float(eps), _ptr(state),
+            _ptr(step.row_start), _ptr(step.state_slots), _ptr(la), _ptr(gate), _ptr(out), _code(out.dtype), T, step.num_rows, whole,
+            H, G, d, dv, chunks, dp, vp, _ptr(scratch), self._stream()))
         return out
 
     GLA_CHUNK = 64           # tokens a chunk of the gated linear attention's scan; rows up to this long run whole
@@ -1488,8 +1559,9 @@ class HipBackend(KernelBackend):
         only_kept = kept and not (sigmoid or softcap is not None or chunk is not None or distance_bias is not None)
         if kept and not only_kept:
             force_generic, biased = True, False     # kept keys or sinks a head beside another variation: the 32-bit kernel
-        if scored and not sigmoid and not biased and not only_kept:
-            force_generic = True            # a capped or chunked softmax: the 32-bit kernel computes it
+        only_chunked = chunk is not None and not (sigmoid or softcap is not None or distance_bias is not None or kept or has_sink)
+        if scored and not sigmoid and not biased and not only_kept and not only_chunked:
+            force_generic = True            # a capped softmax, or chunks beside another variation: the 32-bit kernel computes it
         table2 = None
         if biased and qkv.dtype == torch.bfloat16 and not force_generic and D <= 256:
             # the matrix-core kernels work in units of log2 e: the table in those units, made once a table
@@ -1497,7 +1569,7 @@ class HipBackend(KernelBackend):
         sinks2 = self._in_log2(head_sinks) if head_sinks is not None and qkv.dtype == torch.bfloat16 and not force_generic and D <= 256 else None
         if isinstance(qkv, ProjectionSums):
             out = self._decode_attention_from_sums(qkv, Hq, Hkv, D, k_cache, v_cache, group, step, scale, window,
-                                                   force_generic or num_splits is not None or bool(has_sink) or kept)
+                                                   force_generic or num_splits is not None or bool(has_sink) or kept or chunk is not None)
             if out is not None:
                 return out
             qkv = qkv.finish()
@@ -1530,6 +1602,8 @@ class HipBackend(KernelBackend):
             if sigmoid:
                 library.check(lib, lib.mie_decode_attention_sigmoid(*args, int(chunk or 0), float(softcap or 0.0),
                                                                     _ptr(head_bias), self._stream()))
+            elif only_chunked:
+                library.check(lib, lib.mie_decode_attention_chunked(*args, int(chunk), self._stream()))
             elif kept:
                 library.check(lib, lib.mie_decode_attention_kept(*args, keep_first, _ptr(sinks2), self._stream()))
             elif table2 is not None:
@@ -1553,6 +1627,8 @@ class HipBackend(KernelBackend):
             if sigmoid:
                 library.check(lib, lib.mie_prefill_attention_sigmoid(*args, int(chunk or 0), float(softcap or 0.0),
                                                                      _ptr(head_bias), self._stream()))
+            elif only_chunked:
+                library.check(lib, lib.mie_prefill_attention_chunked(*args, int(chunk), self._stream()))
             elif kept:
                 library.check(lib, lib.mie_prefill_attention_kept(*args, keep_first, _ptr(sinks2), self._stream()))
             elif table2 is not None:

@@ -10,7 +10,8 @@ P, I, L, F = c_void_p, c_int, c_long, c_float
 _head_variants = [(f"-DHEAD_DIM={d}",) for d in HEAD_DIMS]
 
 register_kernel_module("embed_norm", {
-    "mie_embedding": [P, P, I, P, I, I, I, P, P, F, P],
+    "mie_embedding": [P, P, I, P, I, I, I, P, P, F, P, I, L, P],
+    "mie_stream_copy": [P, I, P, P, P, I, L, I, I, P],
     "mie_add_rmsnorm": [P, I, P, P, I, P, I, P, I, I, F, P],
     "mie_branch_norm_add": [P, I, P, P, I, P, I, I, I, F, P],
     "mie_rmsnorm_columns": [P, L, P, I, P, I, I, I, F, P],
@@ -20,7 +21,7 @@ register_kernel_module("embed_norm", {
     "mie_branch_norm_conv_single": [P, P, P, F, P, P, P, P, P, I, I, I, I, F, P],
 })
 register_kernel_module("layer_norm", {
-    "mie_add_layernorm": [P, I, P, P, P, P, I, P, I, I, F, P],
+    "mie_add_layernorm": [P, I, P, P, P, P, P, I, P, I, I, F, P],
     "mie_branch_layernorm_add": [P, I, P, P, P, F, P, P, F, P, I, I, I, P],
     "mie_scale_softcap": [P, L, F, F, P],
 })
@@ -40,7 +41,7 @@ register_kernel_module("grouped_gemm", {
     "mie_grouped_linear": [P, I, L, L, I, P, I, L, L, P, I, L, L, P, P, L, P, P, I, I, I, I, I, I, P, P],
     "mie_grouped_glu": [P, I, L, P, I, L, L, P, I, L, P, P, I, I, I, I, I, F, F, F, P, P],
     "mie_route_topk": [P, L, P, P, P, I, I, I, P],
-    "mie_route_topk_all": [P, L, P, P, P, P, I, I, I, I, P],
+    "mie_route_topk_all": [P, L, P, P, P, P, I, I, I, I, I, F, P],
     "mie_moe_align": [P, I, I, P, P, P, P],
     "mie_moe_combine": [P, P, P, P, I, I, I, P],
     "mie_moe_combine_identity": [P, P, P, P, I, I, I, P, I, P, I, L, P],
@@ -55,16 +56,20 @@ register_kernel_module("recurrence", {
     "mie_rglru_scan_chunked": [P, P, P, P, L, P, P, L, P, P, P, P, P, P, I, I, I, I, F, I, I, P, P, P, P],
     "mie_residual_conv": [P, P, P, P, P, P, P, I, I, I, I, I, P],
     "mie_short_conv": [P, L, P, P, P, P, P, P, P, I, I, I, I, I, P],
-    "mie_conv_tail_move": [P, L, P, P, P, I, I, I, P],
+    "mie_conv_tail_move": [P, L, P, P, P, P, I, I, I, P],
 })
 register_kernel_module("attention_prep", {
     "mie_qkv_finish": [P, L, I, I, I, P, P, F, I, P, I, I, P, P, P, P, P, P, I, I, I, I, I, I, I, I, P, F, I, P],
     "mie_head_gate": [P, I, P, L, I, I, I, P],
-    "mie_qkv_conv_finish": [P, L, I, P, P, P, P, P, I, I, P, P, F, P, I, F, P, P, P, P, F, P, P, P, I, I, I, I, I, I, I, I, P],
+    "mie_qkv_conv_finish": [P, L, I, P, P, P, P, P, P, I, I, P, P, F, I, P, I, I, F, P, P, P, P, F, P, P, P, I, I, I, I, I, I, I, I, P],
     "mie_gate_heads": [P, I, P, L, P, L, I, I, I, I, F, P],
 })
 register_kernel_module("delta_rule", {
     "mie_delta_rule": [P, L, I, I, I, I, I, I, P, I, P, F, P, P, F, P, P, P, P, P, I, I, I, I, I, I, I, P, P, P],
+})
+register_kernel_module("gated_delta", {
+    "mie_gated_delta": [P, L, I, I, I, P, L, I, I, I, P, I, P, P, P, I, F, P, F, P, P, P, P, P, P, I, I, I, I, I, I, I, I, I, I, I, P, P],
+    "mie_gated_delta_unit_floats": [I, I],
 })
 register_kernel_module("gla", {
     "mie_gla": [P, L, I, I, I, I, I, P, I, P, F, F, P, F, P, P, P, P, P, I, I, I, I, I, I, I, I, P, P, P, P],
@@ -99,6 +104,7 @@ register_kernel_module("attention_bf16", {
     "mie_decode_attention_sigmoid": [P, L, P, P, P, P, P, P, I, P, I, I, I, I, I, F, I, I, I, I, F, P, P],
     "mie_decode_attention_biased": [P, L, P, P, P, P, P, P, I, P, I, I, I, I, I, F, I, I, I, P, I, P],
     "mie_decode_attention_kept": [P, L, P, P, P, P, P, P, I, P, I, I, I, I, I, F, I, I, I, I, P, P],
+    "mie_decode_attention_chunked": [P, L, P, P, P, P, P, P, I, P, I, I, I, I, I, F, I, I, I, I, P],
     "mie_decode_attention_from_sums": [P, I, L, L, P, P, P, P, P, P, P, I, P, I, I, I, I, I, F, I, I, P],
     "mie_decode_attention_static": [P, L, P, P, P, P, I, P, I, I, I, I, I, F, I, I, I, P],
     "mie_decode_attention_static_setup": [],
@@ -113,6 +119,7 @@ register_kernel_module("prefill_attention_bf16", {
     "mie_prefill_attention_sink": [P, L, P, P, P, P, I, P, P, I, I, I, I, I, I, I, F, I, F, P],
     "mie_prefill_attention_sigmoid": [P, L, P, P, P, P, I, P, P, I, I, I, I, I, I, I, F, I, I, F, P, P],
     "mie_prefill_attention_biased": [P, L, P, P, P, P, I, P, P, I, I, I, I, I, I, I, F, I, P, I, P],
+    "mie_prefill_attention_chunked": [P, L, P, P, P, P, I, P, P, I, I, I, I, I, I, I, F, I, I, P],
     "mie_prefill_attention_kept": [P, L, P, P, P, P, I, P, P, I, I, I, I, I, I, I, F, I, I, P, P],
 }, variants=_head_variants, flags=["-mllvm", "-amdgpu-mfma-vgpr-form"])
 # lt_gemm: host code only, the engine's own way into the library's matrix products (hipBLASLt) with the choice of

@@ -47,6 +47,8 @@ class Decoder:
                 ce.group = group_keys.index(key)
             self.cache_entries[e] = ce
         self.bindings: list[CacheBinding] = []
+        # parts that run before a layer call (an entry that runs before several is one part)
+        self.entries = list({id(call.entry): call.entry for call in spec.schedule if call.entry is not None}.values())
         # whether a step may carry padding tokens (written to the scratch page): not if a mixer keeps state that
         # every token of a row changes
         self.padding_safe = not any(ce.requirement.stateful for ce in self.cache_entries.values())
@@ -54,7 +56,7 @@ class Decoder:
     # ------------------------------------------------------------ structure
     def parts(self):
         seen = set()
-        roots = [self.spec.embedding, *self.spec.layers, self.spec.final_norm, self.spec.head]
+        roots = [self.spec.embedding, *self.entries, *self.spec.layers, self.spec.final_norm, self.spec.head]
         for r in roots:
             for p in r.walk():
                 if id(p) not in seen:
@@ -111,11 +113,20 @@ class Decoder:
         """Runs exactly the tokens of ``step`` and returns logits [wanted, vocab] in
         32-bit for ``step.logit_rows`` (flat token positions)."""
         spec = self.spec
-        residual = spec.embedding.forward(step.input_ids, step.taken_from, step.earlier_tokens)
+        if self.entries:        # they read what the embedding leaves, beside the stream as it is then
+            copy = self.entries[0].keep_embedding(step, spec.embedding.width)
+            residual = spec.embedding.forward(step.input_ids, step.taken_from, step.earlier_tokens, copy=copy)
+        else:
+            residual = spec.embedding.forward(step.input_ids, step.taken_from, step.earlier_tokens)
         h = None
         last = len(spec.schedule) - 1
         for e, (call, binding) in enumerate(zip(spec.schedule, self.bindings)):
-            after = spec.final_norm if e == last else spec.layers[spec.schedule[e + 1].layer].first_norm
+            if call.entry is not None:
+                h, residual = call.entry.forward(h, residual, step, call.turn)
+            if e == last:
+                after = spec.final_norm
+            else:               # an entry reads the stream itself, not a norm of it
+                after = None if spec.schedule[e + 1].entry is not None else spec.layers[spec.schedule[e + 1].layer].first_norm
             h, residual = spec.layers[call.layer].forward(h, residual, step, binding, next_norm=after)
         if step.num_logits == 0:
             return None

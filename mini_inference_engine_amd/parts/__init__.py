@@ -7,10 +7,12 @@ from .block import BranchNormBlock, ParallelBlock, PreNormBlock, SandwichBlock
 from .delta_rule import DeltaRule
 from .dense_ff import DenseFF
 from .embedding import Embedding, LMHead
+from .gated_delta import GatedDelta
 from .gla import GatedLinearAttention
 from .input_conv import ConvTail, ResidualConv
 from .latent_attention import LatentAttention, PagedLatent
 from .layernorm import LayerNorm
+from .loop_entry import LoopEntry
 from .mlstm import MatrixLSTM, MatrixMemory
 from .rglru import RGLRU, RecurrentState
 from .rmsnorm import RMSNorm

@@ -388,9 +388,12 @@ def register_block(kind: str):
 class LayerCall:
     """One entry of the run order: which layer runs, and whose cache it uses.
     ``cache_of`` names an earlier entry of the run order whose cache this call
-    reads instead of owning one."""
+    reads instead of owning one.  ``entry`` (a parts.LoopEntry): runs right before the
+    layer, for its pass number ``turn``."""
     layer: int
     cache_of: int | None = None
+    entry: Any = None
+    turn: int = 0
 
 
 @dataclass

@@ -23,8 +23,11 @@ class Embedding(Part):
     def params(self):
         return [ParamSpec.single("weight", self.weight_name, (self.vocab_size, self.width))]
 
-    def forward(self, ids, taken_from=None, earlier_tokens=None):
-        """``taken_from`` / ``earlier_tokens``: see KernelBackend.embedding (tokens still on the device)."""
+    def forward(self, ids, taken_from=None, earlier_tokens=None, copy=None):
+        """``taken_from`` / ``earlier_tokens``: see KernelBackend.embedding (tokens still on the device).  ``copy``: a second
+        place for the rows, in the activation dtype."""
+        if copy is not None:
+            return self.ops.embedding(ids, self.weight, taken_from, earlier_tokens, scale=self.scale, copy=copy)
         if self.scale != 1.0:
             return self.ops.embedding(ids, self.weight, taken_from, earlier_tokens, scale=self.scale)
         return self.ops.embedding(ids, self.weight, taken_from, earlier_tokens)

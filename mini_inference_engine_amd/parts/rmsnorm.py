@@ -8,7 +8,7 @@ the weights are loaded).  The stream and every intermediate are 32-bit; y is rou
 """
 from __future__ import annotations
 
-from ..kernels.api import Normed, NormedBranch, StreamCopy
+from ..kernels.api import BiasedBranch, Normed, NormedBranch, StreamCopy
 from .base import Norm, ParamSpec, register_norm
 
 
@@ -41,10 +41,13 @@ class RMSNorm(Norm):
             x = None
         if isinstance(x, StreamCopy):       # the block before left nothing pending
             x = None
+        if isinstance(x, BiasedBranch):     # a branch whose bias is still to be added: both are, now
+            residual.add_(x.float())
+            x = None
         return Normed(self.ops, x, residual, self.weight, self.eps, rows)
 
     def forward(self, x, residual, rows=None, out_dtype=None):
-        if isinstance(x, (Normed, NormedBranch, StreamCopy)):
+        if isinstance(x, (BiasedBranch, Normed, NormedBranch, StreamCopy)):
             return self.lazy(x, residual, rows).materialize(out_dtype)
         return self.ops.add_rmsnorm(x, residual, self.weight, self.eps, out_dtype=out_dtype, rows=rows)
 

@@ -112,15 +112,19 @@ class RotaryHalfAngles(RotaryInterleaved):
 
 
 @register_position_encoding("rotary_yarn")
-class RotaryYarn(RotaryHalfAngles):
-    """The halves' pairing with frequencies stretched by parts (YaRN: Peng et al., "YaRN: Efficient Context Window
+class RotaryYarn(RotaryInterleaved):
+    """Either pairing (``layout``: "half", the default, or "interleaved") with frequencies stretched by parts (YaRN: Peng et al., "YaRN: Efficient Context Window
     Extension of Large Language Models").  With n(t) = rotary_dim ln(original / (2 pi t)) / (2 ln theta), the place of the
     pair that turns t times over ``original`` positions: pairs up to floor(n(fast)) keep their frequency, pairs from
     ceil(n(slow)) on have theirs divided by ``factor``, those between move from one to the other linearly.  Cosines
     and sines are multiplied by 0.1 ln(factor) + 1."""
 
-    def __init__(self, rotary_dim: int, theta: float, factor: float, original: float, fast: float, slow: float):
+    def __init__(self, rotary_dim: int, theta: float, factor: float, original: float, fast: float, slow: float,
+                 layout: str = "half"):
         super().__init__(rotary_dim, theta)
+        if layout not in ("half", "interleaved"):
+            raise ValueError(f"layout {layout!r} (interleaved or half)")
+        self.layout = layout
         self.stretch, self.original, self.fast, self.slow = float(factor), float(original), float(fast), float(slow)
         if not (self.stretch > 0 and self.original > 0 and self.fast > 0 and self.slow > 0) or self.theta == 1.0:
             raise ValueError("factor, original, fast and slow must be positive, and theta another number than 1")

@@ -1,10 +1,12 @@
 """Feed-forward of routed experts: each token runs the ``top`` experts its router prefers.
 
-Router logits z = W_r x (+ b_r) in 32-bit.  Two ways from logits to choice and shares:
+Router logits z = W_r x (+ b_r) in 32-bit.  Three ways from logits to choice and shares:
   ``shares_over="chosen"``  the ``top`` largest logits are chosen; shares are the softmax over those alone;
   ``shares_over="all"``     scores s = softmax(z) over every router output; chosen are the ``top`` largest of
                             s + c (``choice_bias``: a checkpoint vector c that steers the choice only); shares are the
-                            chosen outputs' s, not renormalised, or, with ``renormalise``, divided by their sum + 1e-20.
+                            chosen outputs' s, not renormalised, or, with ``renormalise``, divided by their sum + 1e-20;
+  ``shares_over="sigmoid"`` the same with scores s = sigmoid(z), every output by itself.
+``share_scale`` is a factor on the shares of the latter two.
 An expert is W_down act(W_up x) without biases (act: the square of relu unless another of kernels.api.ACTIVATIONS
 is named), or, with ``gated=(limit, alpha)``, W_down (g * sigmoid(alpha g) * (u + 1)) with g = min(W_gate x, limit)
 and u = clamp(W_up x, -limit, limit); ``gated=(limit, alpha, shift)`` adds ``shift`` to u instead of 1, and
@@ -22,22 +24,23 @@ from .base import FeedForward, ParamSpec, register_feed_forward
 class RoutedExperts(FeedForward):
     def __init__(self, width: int, inner: int, num_experts: int, top: int, prefix: str, activation: str = "relu2",
                  router_bias: bool = True, tensor_names=None, shares_over: str = "chosen", choice_bias: bool = False,
-                 gated=None, identity: int = 0, renormalise: bool = False):
+                 gated=None, identity: int = 0, renormalise: bool = False, share_scale: float = 1.0):
         from ..kernels.api import ACTIVATIONS
         if activation not in ACTIVATIONS:
             raise ValueError(f"activation {activation!r}: one of {ACTIVATIONS}")
-        if shares_over not in ("chosen", "all"):
-            raise ValueError(f"shares_over {shares_over!r}: chosen or all")
+        if shares_over not in ("chosen", "all", "sigmoid"):
+            raise ValueError(f"shares_over {shares_over!r}: chosen, all or sigmoid")
         if identity < 0 or num_experts < 0 or not 1 <= top <= num_experts + identity:
             raise ValueError(f"top {top} of {num_experts} experts and {identity} identity outputs")
-        if choice_bias and shares_over != "all":
-            raise ValueError("a choice bias steers the choice among scores over all outputs (shares_over='all')")
+        if (choice_bias or share_scale != 1.0) and shares_over == "chosen":
+            raise ValueError("a choice bias and a factor on the shares go with scores over all outputs (shares_over 'all' or 'sigmoid')")
         self.width, self.inner, self.num_experts, self.top = int(width), int(inner), int(num_experts), int(top)
         self.identity = int(identity)
         self.prefix, self.activation, self.router_bias = prefix, activation, bool(router_bias)
         self.shares_over, self.has_choice_bias = shares_over, bool(choice_bias)
-        if renormalise and shares_over != "all":
-            raise ValueError("shares over the chosen outputs alone already sum to one (renormalise goes with shares_over='all')")
+        if renormalise and shares_over == "chosen":
+            raise ValueError("shares over the chosen outputs alone already sum to one (renormalise goes with 'all' and 'sigmoid')")
+        self.share_scale = float(share_scale)
         self.renormalise = bool(renormalise)
         if gated == "silu":
             gated = (float("inf"), 1.0, 0.0)
@@ -83,12 +86,11 @@ class RoutedExperts(FeedForward):
         import torch
         ops, E = self.ops, self.num_experts
         logits = ops.linear(x, self.w_router, out_dtype=torch.float32)
-        if self.renormalise:
-            experts, shares = ops.route_topk(logits, self.b_router if self.router_bias else None, self.top,
-                                             over=self.shares_over, choice_bias=self.choice_bias, renormalise=True)
-        else:
-            experts, shares = ops.route_topk(logits, self.b_router if self.router_bias else None, self.top,
-                                             over=self.shares_over, choice_bias=self.choice_bias)
+        opts = dict(renormalise=True) if self.renormalise else {}
+        if self.share_scale != 1.0:
+            opts["scale"] = self.share_scale
+        experts, shares = ops.route_topk(logits, self.b_router if self.router_bias else None, self.top,
+                                         over=self.shares_over, choice_bias=self.choice_bias, **opts)
         rows = self.inner if self.gated is None else 2 * self.inner
         w_up = None if not E else self.w_up.view(E, rows, self.width)
         w_down = None if not E else self.w_down.view(E, self.width, self.inner)

@@ -26,17 +26,23 @@ concatenated heads are multiplied number by number with sigmoid(W_g h).  ``share
 layer leaves its values in ``step.shared`` for later layers of the step / caches (1 - lambda) v + lambda v_shared instead of
 its own values v, lambda a checkpoint number (the layer that leaves them has one too, which nothing reads).
 
+``qk_norm`` "turned": queries and keys are divided head by head by their root mean square after the rotation, without
+weights.  ``chunk``: a query sees the earlier keys of its own chunk only, floor(i / chunk) = floor(j / chunk), chunks counted
+from the request's first position (pages that lie wholly before the chunk of a request's next token are given back: the cache
+sees the chunk as a window of that many keys, which no chunk exceeds).  ``out_bias``: the output projection has a bias.
+
 Keys and queries of ``dim`` and values of ``vdim`` numbers a head are kept in a cache of P = the next multiple of
 16 of the larger one, zeros beyond their own size, so that every head size runs the same attention kernels; the
 output projection's columns are spread to match when the weights are loaded.
 """
 from __future__ import annotations
 
+from ..kernels.api import BiasedBranch, Sink
 from .base import CombinedCache, Mixer, PagedKV, ParamSpec, register_mixer
 from .input_conv import ConvTail
 
 DEFAULT_NAMES = dict(q="q", k="k", v="v", g="g", o="o", temp="temp", q_norm="q.norm", k_norm="k.norm", q_bias="q.b",
-                     k_bias="k.b", v_bias="v.b", distance_bias="rel", q_conv="q.conv", k_conv="k.conv", v_conv="v.conv",
+                     k_bias="k.b", v_bias="v.b", o_bias="o.b", distance_bias="rel", q_conv="q.conv", k_conv="k.conv", v_conv="v.conv",
                      sink="sink", value_mix="vmix")
 
 
@@ -64,7 +70,8 @@ class SoftmaxAttention(Mixer):
                  head_temperature: bool = False, head_gate: bool = False, qk_norm=False, eps: float = 1e-6,
                  float32_output: bool = False, tensor_names=None, bias: bool = False, position_temperature=None,
                  distance_bias=None, conv: int | None = None, keep_first: int = 0, element_gate: bool = False,
-                 share_values: str | None = None, take_values: str | None = None):
+                 share_values: str | None = None, take_values: str | None = None, chunk: int | None = None,
+                 out_bias: bool = False):
         if num_heads % num_kv_heads:
             raise ValueError(f"{num_heads} query heads are not a multiple of {num_kv_heads} kv heads")
         if values_from_keys and vdim != dim:
@@ -79,21 +86,23 @@ class SoftmaxAttention(Mixer):
         if self.padded_dim > 1024:
             raise ValueError(f"heads of {max(dim, vdim)} numbers are beyond the 1024 the attention kernels take")
         self.position, self.prefix = position, prefix
-        self.window = window
+        if chunk is not None and chunk < 1:
+            raise ValueError("chunk must be >= 1 or None")
+        self.window, self.chunk = window, chunk
         self.head_sink = sink == "head"
         self.sink = None if sink is None or self.head_sink else float(sink)
         self.values_from_keys, self.head_temperature = bool(values_from_keys), bool(head_temperature)
-        if qk_norm not in (False, True, "head"):
-            raise ValueError(f"qk_norm {qk_norm!r}: False, True (the whole projection) or 'head'")
-        self.head_gate, self.qk_norm, self.eps = bool(head_gate), bool(qk_norm), float(eps)
+        if qk_norm not in (False, True, "head", "turned"):
+            raise ValueError(f"qk_norm {qk_norm!r}: False, True (the whole projection), 'head' or 'turned' (after the rotation)")
+        self.norm_turned = qk_norm == "turned"
+        self.head_gate, self.qk_norm, self.eps = bool(head_gate), bool(qk_norm) and not self.norm_turned, float(eps)
         self.norm_per_head = qk_norm == "head"
         self.element_gate = bool(element_gate)
         if self.element_gate and self.head_gate:
             raise ValueError("one output gate: per head or per number")
         self.conv = None if conv is None else int(conv)
-        if self.conv is not None and (self.conv < 1 or self.values_from_keys or bias):
-            raise ValueError("a convolution on the projections has at least one tap, and is not built with biases or with "
-                             "values that are the keys")
+        if self.conv is not None and (self.conv < 1 or self.values_from_keys):
+            raise ValueError("a convolution on the projections has at least one tap, and is not built with values that are the keys")
         self.keep_first = int(keep_first)
         if self.keep_first < 0 or (self.keep_first and window is None):
             raise ValueError(f"keep_first {keep_first} belongs beside a window")
@@ -101,15 +110,16 @@ class SoftmaxAttention(Mixer):
         if (share_values or take_values) and (self.values_from_keys or (share_values and take_values)):
             raise ValueError("a layer leaves its own values or takes another's, and projects them itself")
         self.has_taps = self.conv is not None
-        if self.conv is None and (share_values or take_values or (position is not None and position.magnitude != 1.0)):
-            if bias or head_temperature or position_temperature is not None or (qk_norm and not self.norm_per_head):
-                raise ValueError("a scaled rotation and shared values are built with norms head by head, without biases and temperatures")
+        if self.conv is None and (share_values or take_values or self.norm_turned or (position is not None and position.magnitude != 1.0)):
+            if head_temperature or position_temperature is not None or (self.qk_norm and not self.norm_per_head):
+                raise ValueError("a scaled rotation, norms after it and shared values are built with norms head by head, without temperatures")
             self.conv = 1           # built for convolved projections only: one tap of one leaves them as they are
         self.taps = self.value_mix = None
         self.mix = 0.0
         self.float32_output = bool(float32_output)
         self.names = dict(DEFAULT_NAMES, **(tensor_names or {}))
-        self.has_bias = bool(bias)
+        self.has_bias, self.out_bias = bool(bias), bool(out_bias)
+        self.b_o = None
         self.position_temperature = None
         if position_temperature is not None:
             coef, every = float(position_temperature[0]), int(position_temperature[1])
@@ -158,12 +168,15 @@ class SoftmaxAttention(Mixer):
                 raise ValueError("biased projections with values that are the keys are not built")
             specs.append(ParamSpec.stacked("b_in", [(name("q_bias"), (H * self.dim,)), (name("k_bias"), (G * self.dim,)),
                                                     (name("v_bias"), (G * self.vdim,))]))
+        if self.out_bias:
+            specs.append(ParamSpec.single("b_o", name("o_bias"), (w,)))
         if self.distance_buckets is not None:
             specs.append(ParamSpec.single("rel", name("distance_bias"), (self.num_buckets, H)))
         return specs
 
     def cache_requirement(self):
-        kv = PagedKV(self.num_kv_heads, self.padded_dim, self.window, self.keep_first)
+        reach = min((n for n in (self.window, self.chunk) if n is not None), default=None)
+        kv = PagedKV(self.num_kv_heads, self.padded_dim, reach, self.keep_first)
         return kv if self.conv is None else CombinedCache([("kv", kv), ("conv", ConvTail(self.channels, self.conv))])
 
     def prepare(self, device, dtype):
@@ -181,7 +194,7 @@ class SoftmaxAttention(Mixer):
             spread = torch.zeros((self.width, H, P), dtype=self.w_o.dtype, device=self.w_o.device)
             spread[:, :, :self.vdim] = self.w_o.view(self.width, H, self.vdim)
             self.w_o = spread.view(self.width, H * P)
-        for attr in ("temperature", "q_norm", "k_norm", "taps") + (("sink",) if self.head_sink else ()):     # 32-bit whatever the checkpoint stores
+        for attr in ("temperature", "q_norm", "k_norm", "taps", "b_o") + (("sink",) if self.head_sink else ()):     # 32-bit whatever the checkpoint stores
             if getattr(self, attr, None) is not None:
                 setattr(self, attr, getattr(self, attr).float().contiguous())
         if self.conv is not None and not self.has_taps:
@@ -205,6 +218,8 @@ class SoftmaxAttention(Mixer):
             opts["position_temperature"] = self.position_temperature
         if self.norm_per_head:
             opts["norm_per_head"] = True
+        if self.norm_turned:
+            opts["norm_turned"] = True
         if self.position is not None and self.position.magnitude != 1.0:
             opts["rotation_scale"] = self.position.magnitude
         return opts
@@ -238,6 +253,8 @@ class SoftmaxAttention(Mixer):
             more["distance_bias"] = self.distance_table
         if self.keep_first:
             more["keep_first"] = self.keep_first
+        if self.chunk is not None:
+            more["chunk"] = self.chunk
         return ops.paged_attention(q, H, G, P, cache.k, cache.v, group, step, self.scale, self.window, sink=self.sink, **more)
 
     @property
@@ -248,8 +265,8 @@ class SoftmaxAttention(Mixer):
     def branch_into(self, out, scale, sums, base, step, cache):
         """What the output matrix reads, times ``scale``, into ``out`` [T, branch_width] (a caller that joins several
         parts' outputs in one product); ``sums``, ``base`` as for forward."""
-        if not self.element_gate:
-            raise ValueError("joining outputs is built for heads with a gate per number")
+        if not self.element_gate or self.out_bias:
+            raise ValueError("joining outputs is built for heads with a gate per number and no output bias")
         o = self._attend(sums, base, step, cache)
         self.ops.gate_heads(o, sums, base + self.gate_col, self.num_heads, self.vdim, self.padded_dim, out=out, scale=scale)
 
@@ -267,6 +284,11 @@ class SoftmaxAttention(Mixer):
             o = ops.head_gate_(o, sums, base + self.gate_col, H, P)
         elif self.element_gate:
             o = ops.gate_heads(o, sums, base + self.gate_col, H, self.vdim, P)
+        if self.out_bias:
+            if add_to is None:
+                return ops.linear(o, self.w_o, out_dtype=torch.float32).add_(self.b_o)
+            y = ops.linear(o, self.w_o, add_to=Sink(add_to.stream) if isinstance(add_to, Sink) else add_to)
+            return BiasedBranch(y, self.b_o)        # the bias is added by whoever reads the stream next
         if add_to is None and self.float32_output:
             return ops.linear(o, self.w_o, out_dtype=torch.float32)
         return ops.linear(o, self.w_o, add_to=add_to)

@@ -126,16 +126,16 @@ def ref_rglru_scan(u, gates, lam, y, y_col, y_bias, x, x_col, x_bias, state, tai
     return out.to(out_dtype)
 
 
-def ref_route_topk(logits, bias, top, over="chosen", choice_bias=None, renormalise=False):
+def ref_route_topk(logits, bias, top, over="chosen", choice_bias=None, renormalise=False, scale=1.0):
     z = logits.double() if bias is None else logits.double() + bias.double()
-    if over == "all":
-        scores = torch.softmax(z.float(), -1).double()
+    if over in ("all", "sigmoid"):
+        scores = (torch.softmax(z.float(), -1) if over == "all" else torch.sigmoid(z.float())).double()
         by = scores if choice_bias is None else (scores.float() + choice_bias.float()).double()
         idx = torch.sort(by, dim=-1, descending=True, stable=True).indices[:, :top]
         shares = torch.gather(scores, 1, idx)
         if renormalise:
             shares = shares / (shares.sum(-1, keepdim=True) + 1e-20)
-        return idx.to(torch.int32), shares.float()
+        return idx.to(torch.int32), (shares * scale).float()
     order = torch.sort(z, dim=-1, descending=True, stable=True)
     idx, val = order.indices[:, :top], order.values[:, :top]
     return idx.to(torch.int32), torch.softmax(val, -1).float()
@@ -278,15 +278,15 @@ def ref_turn(x, positions, inv_freq, layout):
 
 def ref_qkv_finish(sums, q_col, k_col, v_col, Hq, Hkv, dim, vdim, P, positions, inv_freq, layout, k_cache, v_cache, slots,
                    q_norm, k_norm, eps, q_head_scale, out_dtype, norm_per_head=False, col_bias=None, position_temperature=None,
-                   rotation_scale=1.0, conv=None, values_out=None, value_mix=None):
+                   rotation_scale=1.0, conv=None, values_out=None, value_mix=None, norm_turned=False):
     T = sums.shape[0]
+    if col_bias is not None:
+        sums = (sums.double() + col_bias.double()).float()
     if conv is not None:
         taps, tail, row_start, state_slots = conv
         C = taps.shape[0]
         sums = sums.double()
         sums[:, q_col:q_col + C] = ref_short_conv(sums, q_col, C, taps, None, tail, row_start, state_slots)
-    if col_bias is not None:
-        sums = (sums.double() + col_bias.double()).float()
     q = sums[:, q_col:q_col + Hq * dim].double()
     k = sums[:, k_col:k_col + Hkv * dim].double()
     v = k if v_col is None else sums[:, v_col:v_col + Hkv * vdim].double()
@@ -303,6 +303,9 @@ def ref_qkv_finish(sums, q_col, k_col, v_col, Hq, Hkv, dim, vdim, P, positions, 
         q, k = ref_turn(q, positions, inv_freq, layout), ref_turn(k, positions, inv_freq, layout)
         q[..., :n] *= rotation_scale
         k[..., :n] *= rotation_scale
+    if norm_turned:
+        q = q * torch.rsqrt(q.pow(2).mean(-1, keepdim=True) + eps)
+        k = k * torch.rsqrt(k.pow(2).mean(-1, keepdim=True) + eps)
     if values_out is not None:
         values_out.copy_(v.reshape(T, -1).float())
     if value_mix is not None:
@@ -351,6 +354,40 @@ def ref_delta_rule(sums, cols, H, d, w_decay, decay_bias, decay_scale, removal_b
     return (out.view(T, n) * norm_weight.double() * torch.sigmoid(g.reshape(T, n))).to(out_dtype)
 
 
+def ref_gated_delta(u, q_col, k_col, v_col, sums, beta_col, decay_col, gate_col, H, G, d, dv, w_decay, rate, decay_bias, w_gate, q_scale,
+                    norm_weight, eps, state, row_start, slots, out_dtype):
+    T = u.shape[0]
+    x, s = u.double(), sums.double()
+    unit = lambda t: t * torch.rsqrt(t.pow(2).sum(-1, keepdim=True) + 1e-6)        # noqa: E731
+    q = unit(x[:, q_col:q_col + G * d].view(T, G, d)).repeat_interleave(H // G, 1) * q_scale
+    k = unit(x[:, k_col:k_col + G * d].view(T, G, d)).repeat_interleave(H // G, 1)
+    v = x[:, v_col:v_col + H * dv].view(T, H, dv)
+    beta = torch.sigmoid(s[:, beta_col:beta_col + H])
+    z = s[:, decay_col:decay_col + w_decay.shape[1]] @ w_decay.double().T + decay_bias.double()
+    g = torch.exp(-rate.double()[:, None] * torch.nn.functional.softplus(z, threshold=60).view(T, H, d))
+    gate = torch.sigmoid(s[:, gate_col:gate_col + w_gate.shape[1]] @ w_gate.double().T)
+    out = torch.empty(T, H, dv, dtype=torch.float64, device=u.device)
+    for row in range(len(slots)):
+        S = state[int(slots[row])].double()
+        for t in range(int(row_start[row]), int(row_start[row + 1])):
+            S = g[t][:, :, None] * S
+            w = beta[t][:, None] * (v[t] - torch.einsum("hij,hi->hj", S, k[t]))
+            S = S + k[t][:, :, None] * w[:, None, :]
+            out[t] = torch.einsum("hij,hi->hj", S, q[t])
+        state[int(slots[row])] = S.float()
+    out = out * torch.rsqrt(out.pow(2).mean(-1, keepdim=True) + eps) * norm_weight.double()
+    return (out.view(T, H * dv) * gate).to(out_dtype)
+
+
+def ref_stream_copy(x, stream, x_bias, out):
+    y = stream.double()
+    if x is not None:
+        y = y + x.double()
+    if x_bias is not None:
+        y = y + x_bias.double()
+    return out.copy_(y)
+
+
 def ref_normed_sum_add(stream, ys, weights, eps, scale):
     total = torch.zeros_like(stream, dtype=torch.float64)
     for y, w in zip(ys, weights):
@@ -364,17 +401,22 @@ def ref_layernorm(x, weight, bias, eps):
     xd = x.double()
     mean = xd.mean(-1, keepdim=True)
     var = (xd - mean).pow(2).mean(-1, keepdim=True)
-    return (xd - mean) / torch.sqrt(var + eps) * weight.double() + bias.double()
+    y = (xd - mean) / torch.sqrt(var + eps) * weight.double()
+    return y if bias is None else y + bias.double()
 
 
-def ref_add_layernorm(x, residual, weight, bias, eps, out_dtype, rows=None):
+def ref_add_layernorm(x, residual, weight, bias, eps, out_dtype, rows=None, x_bias=None):
     if rows is not None:
         r = residual[rows.long()].double()
         if x is not None:
             r = r + x[rows.long()].double()
+        if x_bias is not None:
+            r = r + x_bias.double()
         return ref_layernorm(r, weight, bias, eps).to(out_dtype)
     if x is not None:
         residual.add_(x.float())
+    if x_bias is not None:
+        residual.add_(x_bias)
     return ref_layernorm(residual, weight, bias, eps).to(out_dtype)
 
 
@@ -526,11 +568,25 @@ class TorchBackend(KernelBackend):
     def _count(self, name):
         self.calls[name] = self.calls.get(name, 0) + 1
 
-    def embedding(self, ids, table, taken_from=None, earlier_tokens=None, scale=1.0):
+    def embedding(self, ids, table, taken_from=None, earlier_tokens=None, scale=1.0, copy=None):
         self._count("embedding")
         if taken_from is not None:
             ids = torch.where(taken_from >= 0, earlier_tokens[taken_from.clamp(min=0).long()], ids)
-        return ref_embedding(ids, table, scale)
+        rows = ref_embedding(ids, table, scale)
+        if copy is not None:
+            copy.copy_(rows)
+        return rows
+
+    def stream_copy(self, x, stream, out, x_bias=None):
+        self._count("stream_copy")
+        return ref_stream_copy(x, stream, x_bias, out)
+
+    def gated_delta(self, u, q_col, k_col, v_col, sums, beta_col, decay_col, gate_col, num_heads, num_kv_heads, dim, vdim,
+                    w_decay, rate, decay_bias, w_gate, q_scale, norm_weight, eps, state, step):
+        self._count("gated_delta")
+        return ref_gated_delta(u, q_col, k_col, v_col, sums, beta_col, decay_col, gate_col, num_heads, num_kv_heads, dim, vdim, w_decay,
+                               rate, decay_bias, w_gate, q_scale, norm_weight, eps, state, step.host["row_start"],
+                               step.host["state_slots"], self.act_dtype)
 
     def scale_(self, t, factor):
         return t.mul_(factor)
@@ -538,9 +594,9 @@ class TorchBackend(KernelBackend):
     def scale_softcap_(self, t, scale, cap):
         return t.copy_(ref_scale_softcap(t, scale, cap))
 
-    def add_layernorm(self, x, residual, weight, bias, eps, out_dtype=None, rows=None):
+    def add_layernorm(self, x, residual, weight, bias, eps, out_dtype=None, rows=None, x_bias=None):
         self._count("add_layernorm")
-        return ref_add_layernorm(x, residual, weight, bias, eps, out_dtype or self.act_dtype, rows)
+        return ref_add_layernorm(x, residual, weight, bias, eps, out_dtype or self.act_dtype, rows, x_bias)
 
     def branch_layernorm_add(self, y, stream, weight, bias, eps, next_norm=None):
         self._count("branch_layernorm_add")
@@ -598,8 +654,8 @@ class TorchBackend(KernelBackend):
         return ref_rglru_scan(u, gates, lam, y, y_col, y_bias, x, x_col, x_bias, state, tail, step.host["row_start"],
                               step.host["state_slots"], taps, decay_scale, self.act_dtype)
 
-    def route_topk(self, logits, bias, top, over="chosen", choice_bias=None, renormalise=False):
-        return ref_route_topk(logits, bias, top, over, choice_bias, renormalise)
+    def route_topk(self, logits, bias, top, over="chosen", choice_bias=None, renormalise=False, scale=1.0):
+        return ref_route_topk(logits, bias, top, over, choice_bias, renormalise, scale)
 
     def routed_experts(self, x, experts, shares, w_up, w_down, activation="relu2", gated=None, identity_from=None, glu_block=0):
         assert glu_block == 0, "the torch operations keep gate rows before up rows"
@@ -651,13 +707,14 @@ class TorchBackend(KernelBackend):
     def qkv_finish(self, sums, q_col, k_col, v_col, num_q_heads, num_kv_heads, dim, vdim, padded_dim, positions, inv_freq,
                    layout, k_cache, v_cache, slot_mapping, q_norm=None, k_norm=None, eps=0.0, q_head_scale=None,
                    norm_per_head=False, col_bias=None, position_temperature=None, rotation_scale=1.0, conv=None,
-                   values_out=None, value_mix=None):
+                   values_out=None, value_mix=None, norm_turned=False):
         self._count("qkv_finish")
         if conv is not None:
             conv = (conv[0], conv[1], conv[2].host["row_start"], conv[2].host["state_slots"])
         return ref_qkv_finish(sums, q_col, k_col, v_col, num_q_heads, num_kv_heads, dim, vdim, padded_dim, positions, inv_freq,
                               layout, k_cache, v_cache, slot_mapping, q_norm, k_norm, eps, q_head_scale, self.act_dtype,
-                              norm_per_head, col_bias, position_temperature, rotation_scale, conv, values_out, value_mix)
+                              norm_per_head, col_bias, position_temperature, rotation_scale, conv, values_out, value_mix,
+                              norm_turned)
 
     def linear_clamped_glu(self, x, w_gate_up, intermediate, limit, alpha, shift):
         self._count("linear_clamped_glu")
