@@ -3,7 +3,7 @@ Llama-2-7B or Llama-3-8B), random weights.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch 8] [--shape tinyllama] [--context N] [--layers L]
     python bench.py --kernels [--shape ...] [--batch 8] [--context N]     each dominant kernel alone
-    python bench.py --design zifelorn|vezodra|mutusun|labirax|pokulorn [--design-sizes 1024,2048] [--layers R] [--batch 8] [--context 1024]
+    python bench.py --design zifelorn|vezodra|mutusun|labirax|pokulorn|bulitar [--design-sizes 1024,2048] [--layers R] [--batch 8] [--context 1024]
                                                  that design beside Llama at equal layer sizes (R runs of its layers)
 
 A step is one decode step of the engine (schedule, batch, captured forward, sampling,
@@ -483,11 +483,27 @@ POKULORN_SIZES = {
 }
 
 
+# Bulitar layer sizes of the same widths: a run of five layers is the delta rule with a decay a channel once, then two passes of
+# two layers of chunked attention, each pass behind its entry, every layer with experts (four of them a token, together as large
+# as the dense feed-forward).
+BULITAR_SIZES = {
+    "1024": dict(vocab=32000, width=1024, heads=16, kv_heads=4, dim=64, chunk=1024, delta_heads=8, delta_kv_heads=8, delta_dim=128,
+                 delta_vdim=128, rank=128, ff=2816, experts=8, top=4, expert_ff=704),
+    "2048": dict(vocab=32000, width=2048, heads=32, kv_heads=8, dim=64, chunk=1024, delta_heads=16, delta_kv_heads=16, delta_dim=128,
+                 delta_vdim=128, rank=128, ff=5632, experts=16, top=4, expert_ff=1408),
+}
+
+
 def design_configs(design: str, size: str, repeats: int):
     """(the design's configuration, Llama's of the same width, head count, feed-forward size, vocabulary and layer count)."""
-    from mini_inference_engine_amd.config import (LabiraxConfig, LlamaConfig, MutusunConfig, PokulornConfig, VezodraConfig,
+    from mini_inference_engine_amd.config import (BulitarConfig, LabiraxConfig, LlamaConfig, MutusunConfig, PokulornConfig, VezodraConfig,
                                                   ZifelornConfig)
-    if design == "pokulorn":
+    if design == "bulitar":
+        from mini_inference_engine_amd.models.bulitar import _shape
+        z = BULITAR_SIZES[size]
+        cfg = BulitarConfig.from_dict(_shape(repeats=repeats, times=2, **{k: v for k, v in z.items() if k != "ff"}))
+        layers = len(cfg.run_order())
+    elif design == "pokulorn":
         from mini_inference_engine_amd.models.pokulorn import _shape
         z = POKULORN_SIZES[size]
         cfg, layers = PokulornConfig.from_dict(_shape(repeats=repeats, **z)), 3 * repeats
@@ -551,7 +567,7 @@ def measure_designs(args) -> int:
 
 def main() -> int:
     ap = argparse.ArgumentParser()
-    ap.add_argument("--design", choices=["zifelorn", "vezodra", "mutusun", "labirax", "pokulorn"], default=None,
+    ap.add_argument("--design", choices=["zifelorn", "vezodra", "mutusun", "labirax", "pokulorn", "bulitar"], default=None,
                     help="instead of the default workload: that design beside Llama at equal layer sizes (decode and prefill)")
     ap.add_argument("--design-sizes", default=None, help="comma-separated widths of --design (default: all of 1024, 2048)")
     ap.add_argument("--gpus", type=int, default=1)

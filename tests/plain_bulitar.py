@@ -150,10 +150,14 @@ def channel_delta_mixer(h, W, p, m, eps):
 
 
 # ------------------------------------------------------------------ feed-forward
-def choose(h, W, p, top, scale):
-    """-> (experts [n, top], their weights)"""
+def choose(h, W, p, top, scale, margins=None):
+    """-> (experts [n, top], their weights); ``margins`` (a list) gets every token's distance from another choice"""
     s = torch.sigmoid(h @ W[f"{p}.router"].T)
-    picked = torch.topk(s + W[f"{p}.correction"], top, dim=-1).indices
+    by = s + W[f"{p}.correction"]
+    picked = torch.topk(by, top, dim=-1).indices
+    if margins is not None and top < s.shape[-1]:
+        order = by.sort(-1, descending=True).values
+        margins += (order[:, top - 1] - order[:, top]).tolist()
     return picked, torch.gather(s, 1, picked) * scale
 
 
@@ -161,9 +165,9 @@ def expert(x, W, p):
     return (silu(x @ W[f"{p}.gate"].T) * (x @ W[f"{p}.up"].T)) @ W[f"{p}.down"].T
 
 
-def experts_ff(h, W, p, m):
+def experts_ff(h, W, p, m, margins=None):
     r = m["router"]
-    picked, share = choose(h, W, p, r["top"], r["scale"])
+    picked, share = choose(h, W, p, r["top"], r["scale"], margins)
     y = torch.zeros_like(h)
     for t in range(h.shape[0]):
         for j in range(r["top"]):
@@ -186,7 +190,7 @@ def begin_pass(s, first, W, t):
     return torch.cat([s, first], dim=-1) @ W["loop.in"].T + W["loop.step"][t]
 
 
-def forward(config, weights, ids, streams=None, dtype=torch.float64):
+def forward(config, weights, ids, streams=None, dtype=torch.float64, margins=None):
     W = {k: (v.to(dtype) if v.is_floating_point() else v) for k, v in weights.items()}
     eps = config["norm"]["eps"]
     first = W["embed"][torch.as_tensor(ids, dtype=torch.long)] * config["embedding"]["scale"]
@@ -198,7 +202,7 @@ def forward(config, weights, ids, streams=None, dtype=torch.float64):
         mixer = {"attention": attention_mixer, "channel_delta": channel_delta_mixer}[layer["type"]]
         s = s + mixer(layer_norm(s, W[f"{p}.norm1"], eps), W, f"{p}.mix", layer["mixer"], eps)
         if layer.get("mlp") is not None:
-            s = s + experts_ff(layer_norm(s, W[f"{p}.norm2"], eps), W, f"{p}.mlp", layer["mlp"])
+            s = s + experts_ff(layer_norm(s, W[f"{p}.norm2"], eps), W, f"{p}.mlp", layer["mlp"], margins)
         if streams is not None:
             streams.append(s.clone())
     return layer_norm(s, W["final.norm"], eps) @ W["head"].T
