@@ -27,6 +27,12 @@ constexpr float LOG2E = 1.4426950408889634f;
 
 __device__ __forceinline__ float softplus(float z) { return z > 20.f ? z : log1pf(expf(z)); }
 __device__ __forceinline__ float pow2(float x) { return __builtin_amdgcn_exp2f(x); }      // below 2^-126: 0
+// The waves meet over the LDS only: loads and stores of global memory stay on their way (__syncthreads would wait for them)
+__device__ __forceinline__ void lds_barrier() {
+  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+  __builtin_amdgcn_s_barrier();
+  asm volatile("" ::: "memory");
+}
 __device__ __forceinline__ f32x4 mfma4(float a, float b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
 
 // ---- decays and gates: a wave 16 channels of 16 TT tokens.  Operand A lane (n, g): token n, B: channel n; both take inner numbers
@@ -103,7 +109,8 @@ scan_kernel(DeltaArgs a, int CB) {
   float* sg = sk + TB * DP;              // decays
   float* part = sg + TB * DP;            // [2][RG][2][CW]
   float* so = part + 4 * RG * CW;        // [TB][CW]
-  float* sf = so + TB * CW;              // [TB][4]: factors of q and k, k . q, beta
+  float* sv = so + TB * CW;              // [TB][CW]
+  float* sf = sv + TB * CW;              // [TB][4]: factors of q and k, k . q, beta
   const int row = a.first_row + blockIdx.x, h = blockIdx.y, hk = h / a.per_group, col = cb * 64 + lane;
   const int begin = a.row_start[row], end = a.row_start[row + 1];
   const bool active = col < dv;
@@ -124,9 +131,7 @@ scan_kernel(DeltaArgs a, int CB) {
       sk[e] = in ? a.k[at] : 0.f;
       sg[e] = in ? expf(a.la[((size_t)(t0 + tt) * H + h) * d + i]) : 0.f;
     }
-    float v[TB];
-#pragma unroll
-    for (int tt = 0; tt < TB; ++tt) v[tt] = active && tt < nt ? a.v[(size_t)(t0 + tt) * a.ld_u + (size_t)h * dv + col] : 0.f;
+    for (int tt = rg; tt < nt; tt += RG) sv[tt * CW + col] = active ? a.v[(size_t)(t0 + tt) * a.ld_u + (size_t)h * dv + col] : 0.f;
     __syncthreads();
     for (int tt = wave; tt < nt; tt += waves) {
       float qq = 0.f, kk = 0.f, qk = 0.f;
@@ -148,9 +153,8 @@ scan_kernel(DeltaArgs a, int CB) {
       }
     }
     __syncthreads();
-#pragma unroll
-    for (int tt = 0; tt < TB; ++tt) {
-      if (tt >= nt) break;
+#pragma unroll 1
+    for (int tt = 0; tt < nt; ++tt) {
       const float4* q4 = reinterpret_cast<const float4*>(sq + tt * DP + r0);
       const float4* k4 = reinterpret_cast<const float4*>(sk + tt * DP + r0);
       const float4* g4 = reinterpret_cast<const float4*>(sg + tt * DP + r0);
@@ -173,7 +177,7 @@ scan_kernel(DeltaArgs a, int CB) {
         o += mine[(w * 2 + 1) * CW + col];
       }
       buf ^= 1;
-      const float fk = sf[4 * tt + 1], w = sf[4 * tt + 3] * (v[tt] - p * fk), wk = w * fk;
+      const float fk = sf[4 * tt + 1], w = sf[4 * tt + 3] * (sv[tt * CW + col] - p * fk), wk = w * fk;
 #pragma unroll
       for (int i = 0; i < R / 4; ++i) {
         const float4 kk = k4[i];
@@ -205,7 +209,7 @@ scan_kernel(DeltaArgs a, int CB) {
 constexpr int CH = 64, MS = CH + 4;
 struct ChunkArgs {
   DeltaArgs s;
-  int max_chunks, VP;
+  int max_chunks, units, VP;      // units: rows * max_chunks
   float* W;        // [unit][64][DP]
   float* KT;       // [unit][DP][64]   e^(G_end - G_s) k_s, a channel's tokens side by side
   float* QT;       // [unit][64][DP]   e^G_t q_t
@@ -215,15 +219,21 @@ struct ChunkArgs {
   float* ST;       // [unit][DP][VP]   S_0
 };
 
+// Grids run over the heads first: workgroups go to the eight XCDs in turn, so where H is a multiple of 8 all passes of a head run
+// on one XCD and find in its L2 what the pass before left.
 #define CHUNK_OF_ROW                                                                                                    \
-  const int rr = blockIdx.x / p.max_chunks, ci = blockIdx.x - rr * p.max_chunks, row = a.first_row + rr, h = blockIdx.y; \
+  const int place = blockIdx.y + gridDim.y * blockIdx.z;                                                                \
+  if (place >= p.units) return;                                                                                         \
+  const int rr = place / p.max_chunks, ci = place - rr * p.max_chunks, row = a.first_row + rr, h = blockIdx.x;          \
   const int t0 = a.row_start[row] + ci * CH, t_end = a.row_start[row + 1];                                              \
   if (t0 >= t_end) return;                                                                                              \
   const int nt = t_end - t0 < CH ? t_end - t0 : CH;                                                                     \
-  const size_t unit = (size_t)blockIdx.x * a.H + h
+  const size_t unit = (size_t)place * a.H + h
+
+constexpr int SOLVE_THREADS = 512;
 
 template <int DP>
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(SOLVE_THREADS)
 chunk_solve_kernel(ChunkArgs p) {
   constexpr int DS = DP + 4;
   extern __shared__ __align__(16) float lds[];
@@ -233,19 +243,20 @@ chunk_solve_kernel(ChunkArgs p) {
   float* M = sG + CH * DS;           // [64][MS] diag(beta) A, strictly below the diagonal
   float* X = M + CH * MS;            // [64][MS] (I + M)^-1
   float* sb = X + CH * MS;           // [64] beta
+  float* so = sb + CH;               // [4][DP] sums of 16 tokens
   const DeltaArgs& a = p.s;
   CHUNK_OF_ROW;
   const int tid = threadIdx.x, lane = tid & 63, n = lane & 15, g = lane >> 4;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int d = a.d, dv = a.dv, H = a.H, hk = h / a.per_group;
-  // ---- unit vectors and decays into the LDS, a wave 16 tokens, four at a time
+  // ---- unit vectors and decays into the LDS, a wave eight tokens, four at a time
   constexpr int E = (DP + 63) / 64;
 #pragma unroll 1
-  for (int g4 = 0; g4 < 16; g4 += 4) {
+  for (int g4 = 0; g4 < 8; g4 += 4) {
     float q[4][E], k[4][E], l[4][E], qq[4], kk[4];
 #pragma unroll
     for (int u = 0; u < 4; ++u) {
-      const int tt = 16 * wave + g4 + u, t = t0 + (tt < nt ? tt : nt - 1);
+      const int tt = 8 * wave + g4 + u, t = t0 + (tt < nt ? tt : nt - 1);
 #pragma unroll
       for (int e = 0; e < E; ++e) {
         const int i = lane + 64 * e, ic = i < d ? i : d - 1;
@@ -273,7 +284,7 @@ chunk_solve_kernel(ChunkArgs p) {
       }
 #pragma unroll
     for (int u = 0; u < 4; ++u) {
-      const int tt = 16 * wave + g4 + u;
+      const int tt = 8 * wave + g4 + u;
       const float fq = a.q_scale / sqrtf(qq[u] + 1e-6f), fk = 1.0f / sqrtf(kk[u] + 1e-6f);
 #pragma unroll
       for (int e = 0; e < E; ++e) {
@@ -288,58 +299,58 @@ chunk_solve_kernel(ChunkArgs p) {
     }
   }
   if (tid < CH) sb[tid] = tid < nt ? mie_sigmoid(a.beta[(size_t)(t0 + tid) * a.ld + h]) : 0.f;
-  for (int e = tid; e < CH * MS; e += 256) M[e] = X[e] = 0.f;
-  __syncthreads();
-  for (int i = tid; i < DP; i += 256) {
-    float run = 0.f;
-#pragma unroll 16
-    for (int t = 0; t < CH; ++t) {
-      run += sG[t * DS + i];
-      sG[t * DS + i] = run;
-    }
-  }
-  __syncthreads();
-  float* __restrict__ AQ = p.AQ + unit * CH * CH;
-  // ---- pairs within 16 tokens: a wave a block, a lane two tokens t and two tokens s, four channels at a time
+  for (int e = tid; e < CH * MS; e += SOLVE_THREADS) M[e] = X[e] = 0.f;
+  lds_barrier();
+  // ---- sums over the tokens: within 16 tokens, then the 16s before them
   {
-    const int ti = 16 * wave + 2 * (lane >> 3), si = 16 * wave + 2 * (lane & 7);
-    float ak[2][2] = {{0.f, 0.f}, {0.f, 0.f}}, aq[2][2] = {{0.f, 0.f}, {0.f, 0.f}};
-    if (ti >= si) {
-#pragma unroll 2
+    const int i = tid % DP, part = tid / DP;
+    float run = 0.f, at[16];
+    if (part < 4) {
+#pragma unroll
+      for (int t = 0; t < 16; ++t) at[t] = run += sG[(16 * part + t) * DS + i];
+      so[part * DP + i] = run;
+    }
+    lds_barrier();
+    if (part < 4) {
+      float before = 0.f;
+      for (int w = 0; w < part; ++w) before += so[w * DP + i];
+#pragma unroll
+      for (int t = 0; t < 16; ++t) sG[(16 * part + t) * DS + i] = before + at[t];
+    }
+  }
+  lds_barrier();
+  float* __restrict__ AQ = p.AQ + unit * CH * CH;
+  // ---- pairs within 16 tokens: two waves a block, a lane one token t and two tokens s, four channels at a time
+  {
+    const int t = 16 * (wave >> 1) + 2 * (lane >> 3) + (wave & 1), si = 16 * (wave >> 1) + 2 * (lane & 7);
+    float ak[2] = {0.f, 0.f}, aq[2] = {0.f, 0.f};
+    if (t >= si) {
+#pragma unroll 4
       for (int i = 0; i < DP; i += 4) {
-        f32x4 kt[2], qt[2], gt[2], ks[2], gs[2];
+        const f32x4 kt = *reinterpret_cast<const f32x4*>(sk + t * DS + i), qt = *reinterpret_cast<const f32x4*>(sq + t * DS + i);
+        const f32x4 gt = *reinterpret_cast<const f32x4*>(sG + t * DS + i);
 #pragma unroll
-        for (int u = 0; u < 2; ++u) {
-          kt[u] = *reinterpret_cast<const f32x4*>(sk + (ti + u) * DS + i);
-          qt[u] = *reinterpret_cast<const f32x4*>(sq + (ti + u) * DS + i);
-          gt[u] = *reinterpret_cast<const f32x4*>(sG + (ti + u) * DS + i);
-          ks[u] = *reinterpret_cast<const f32x4*>(sk + (si + u) * DS + i);
-          gs[u] = *reinterpret_cast<const f32x4*>(sG + (si + u) * DS + i);
+        for (int w = 0; w < 2; ++w) {
+          const f32x4 ks = *reinterpret_cast<const f32x4*>(sk + (si + w) * DS + i), gs = *reinterpret_cast<const f32x4*>(sG + (si + w) * DS + i);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            const float x = ks[e] * pow2(fminf(gt[e] - gs[e], 0.f));       // a pair above the diagonal is not used
+            ak[w] = fmaf(kt[e], x, ak[w]);
+            aq[w] = fmaf(qt[e], x, aq[w]);
+          }
         }
-#pragma unroll
-        for (int u = 0; u < 2; ++u)
-#pragma unroll
-          for (int w = 0; w < 2; ++w)
-#pragma unroll
-            for (int e = 0; e < 4; ++e) {
-              const float x = ks[w][e] * pow2(fminf(gt[u][e] - gs[w][e], 0.f));       // a pair above the diagonal is not used
-              ak[u][w] = fmaf(kt[u][e], x, ak[u][w]);
-              aq[u][w] = fmaf(qt[u][e], x, aq[u][w]);
-            }
       }
     }
 #pragma unroll
-    for (int u = 0; u < 2; ++u)
-#pragma unroll
-      for (int w = 0; w < 2; ++w) {
-        const int t = ti + u, s = si + w;
-        if (t > s) M[t * MS + s] = sb[t] * ak[u][w];
-        AQ[t * CH + s] = t >= s ? aq[u][w] : 0.f;
-      }
+    for (int w = 0; w < 2; ++w) {
+      const int s = si + w;
+      if (t > s) M[t * MS + s] = sb[t] * ak[w];
+      AQ[t * CH + s] = t >= s ? aq[w] : 0.f;
+    }
   }
-  // ---- tokens of an earlier 16, on the matrix cores: the blocks (x, y) below the diagonal, taken in turn by the waves
-  for (int blk = wave; blk < 6; blk += 4) {
-    const int x = blk < 3 ? 3 : blk < 5 ? 2 : 1, y = blk < 3 ? blk : blk < 5 ? blk - 3 : 0;
+  // ---- tokens of an earlier 16, on the matrix cores: the blocks (x, y) below the diagonal, one a wave
+  if (wave < 6) {
+    const int blk = wave, x = blk < 3 ? 3 : blk < 5 ? 2 : 1, y = blk < 3 ? blk : blk < 5 ? blk - 3 : 0;
     const float* __restrict__ ref = sG + (16 * x - 1) * DS;
     f32x4 acc_k = f32x4{0.f, 0.f, 0.f, 0.f}, acc_q = acc_k;
 #pragma unroll 2
@@ -362,9 +373,9 @@ chunk_solve_kernel(ChunkArgs p) {
       AQ[t * CH + s] = acc_q[e];
     }
   }
-  __syncthreads();
+  lds_barrier();
   // ---- the inverse: diagonal blocks by substitution, a lane a column
-  {
+  if (wave < 4) {
     const float* __restrict__ m = M + 16 * wave * MS + 16 * wave;
     float x[16];
 #pragma unroll
@@ -379,7 +390,7 @@ chunk_solve_kernel(ChunkArgs p) {
       for (int t = 0; t < 16; ++t) X[(16 * wave + t) * MS + 16 * wave + n] = x[t];
     }
   }
-  __syncthreads();
+  lds_barrier();
 #pragma unroll 1
   for (int dist = 1; dist < 4; ++dist) {
     if (wave + dist < 4) {
@@ -398,13 +409,13 @@ chunk_solve_kernel(ChunkArgs p) {
 #pragma unroll
       for (int e = 0; e < 4; ++e) X[(16 * x + 4 * g + e) * MS + 16 * y + n] = -r[e];
     }
-    __syncthreads();
+    lds_barrier();
   }
-  // ---- W and U: a wave every fourth 16 columns
+  // ---- W and U: a wave every eighth 16 columns
   float* __restrict__ W = p.W + unit * CH * DP;
   float* __restrict__ U = p.U + unit * CH * p.VP;
   const int col_tiles = DP / 16 + p.VP / 16;
-  for (int ct = wave; ct < col_tiles; ct += 4) {
+  for (int ct = wave; ct < col_tiles; ct += SOLVE_THREADS / 64) {
     const bool of_w = ct < DP / 16;
     const int c = (of_w ? ct : ct - DP / 16) * 16 + n;
     f32x4 acc[4];
@@ -438,13 +449,13 @@ chunk_solve_kernel(ChunkArgs p) {
   // ---- what the other passes want of keys and queries
   float* __restrict__ KT = p.KT + unit * DP * CH;
   float* __restrict__ QT = p.QT + unit * CH * DP;
-  for (int e = tid; e < CH * DP; e += 256) {
+  for (int e = tid; e < CH * DP; e += SOLVE_THREADS) {
     const int s = e & (CH - 1), i = e / CH;
     KT[e] = sk[s * DS + i] * pow2(sG[(CH - 1) * DS + i] - sG[s * DS + i]);
     const int t = e / DP, j = e % DP;
     QT[e] = sq[t * DS + j] * pow2(sG[t * DS + j]);
   }
-  for (int i = tid; i < DP; i += 256) p.EG[unit * DP + i] = pow2(sG[(CH - 1) * DS + i]);
+  for (int i = tid; i < DP; i += SOLVE_THREADS) p.EG[unit * DP + i] = pow2(sG[(CH - 1) * DS + i]);
 }
 
 // (2) grid (H, rows, VP / 16): the workgroups of a head are H apart, on one XCD where H is a multiple of 8
@@ -468,34 +479,38 @@ chunk_fold_kernel(ChunkArgs p) {
       const int r = 16 * (wave + 4 * i) + 4 * g + e;
       S[i][e] = r < d && col < dv ? st[(size_t)r * dv + col] : 0.f;
     }
-  f32x4 w[KB], kt[RT][4], eg[RT];
-  float u[4];
+  struct Ahead {                          // what a chunk needs, asked for two chunks ahead
+    f32x4 w[KB], kt[RT][4], eg[RT];
+    float u[4];
+  };
   auto unit_of = [&](int c) { return ((size_t)rr * p.max_chunks + c) * H + h; };
-  auto fetch_first = [&](int c) {         // of the first product: W and U
+  auto fetch_first = [&](Ahead& A, int c) {         // of the first product: W and U
+    c = c < chunks ? c : chunks - 1;
     const float* __restrict__ W = p.W + unit_of(c) * CH * DP + (size_t)(16 * wave + n) * DP + 4 * g;
 #pragma unroll
-    for (int kb = 0; kb < KB; ++kb) w[kb] = *reinterpret_cast<const f32x4*>(W + 16 * kb);
+    for (int kb = 0; kb < KB; ++kb) A.w[kb] = *reinterpret_cast<const f32x4*>(W + 16 * kb);
     const float* __restrict__ U = p.U + unit_of(c) * CH * VP + col;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) u[e] = U[(size_t)(16 * wave + 4 * g + e) * VP];
+    for (int e = 0; e < 4; ++e) A.u[e] = U[(size_t)(16 * wave + 4 * g + e) * VP];
   };
-  auto fetch_second = [&](int c) {        // of the second: keys and the chunk's decay
+  auto fetch_second = [&](Ahead& A, int c) {        // of the second: keys and the chunk's decay
+    c = c < chunks ? c : chunks - 1;
 #pragma unroll
     for (int i = 0; i < RT; ++i) {
       const int tile = wave + 4 * i < KB ? wave + 4 * i : KB - 1;
       const float* __restrict__ K = p.KT + unit_of(c) * DP * CH + (size_t)(16 * tile + n) * CH + 4 * g;
 #pragma unroll
-      for (int sb = 0; sb < 4; ++sb) kt[i][sb] = *reinterpret_cast<const f32x4*>(K + 16 * sb);
-      eg[i] = *reinterpret_cast<const f32x4*>(p.EG + unit_of(c) * DP + 16 * tile + 4 * g);
+      for (int sb = 0; sb < 4; ++sb) A.kt[i][sb] = *reinterpret_cast<const f32x4*>(K + 16 * sb);
+      A.eg[i] = *reinterpret_cast<const f32x4*>(p.EG + unit_of(c) * DP + 16 * tile + 4 * g);
     }
   };
-  fetch_first(0);
-  fetch_second(0);
-  for (int c = 0; c < chunks; ++c) {
+  // What a later chunk needs is asked for without a condition (the last chunk's once more at the end): the waits below then count
+  // exactly what was issued since, and never wait for more than they need.
+  auto step = [&](Ahead& A, int c) {
     float* __restrict__ ST = p.ST + unit_of(c) * DP * VP + col;
 #pragma unroll
     for (int i = 0; i < RT; ++i)
-      if (wave + 4 * i < KB) {
+      if (KB % 4 == 0 || wave + 4 * i < KB) {
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
           const int r = 16 * (wave + 4 * i) + 4 * g + e;
@@ -503,32 +518,56 @@ chunk_fold_kernel(ChunkArgs p) {
           ST[(size_t)r * VP] = S[i][e];
         }
       }
-    __syncthreads();
+    lds_barrier();
     f32x4 acc[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
+    float right[KB][4];                   // all of it asked for before the first product
 #pragma unroll
     for (int kb = 0; kb < KB; ++kb)
 #pragma unroll
-      for (int j = 0; j < 4; ++j) acc[kb & 1] = mfma4(w[kb][j], sS[(16 * kb + 4 * g + j) * CS + n], acc[kb & 1]);
+      for (int j = 0; j < 4; ++j) right[kb][j] = sS[(16 * kb + 4 * g + j) * CS + n];
+    asm volatile("" ::: "memory");
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+#pragma unroll
+      for (int kb = 0; kb < KB; ++kb) acc[kb & 1] = mfma4(A.w[kb][j], right[kb][j], acc[kb & 1]);
     float* __restrict__ U = p.U + unit_of(c) * CH * VP + col;
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
       const int t = 16 * wave + 4 * g + e;
-      const float x = u[e] - (acc[0][e] + acc[1][e]);
+      const float x = A.u[e] - (acc[0][e] + acc[1][e]);
       sU[t * CS + n] = x;
       U[(size_t)t * VP] = x;
     }
-    if (c + 1 < chunks) fetch_first(c + 1);
-    __syncthreads();
+    fetch_first(A, c + 2);
+    lds_barrier();
+    float down[4][4];
 #pragma unroll
-    for (int i = 0; i < RT; ++i) {
-      f32x4 s = S[i] * eg[i];
+    for (int sb = 0; sb < 4; ++sb)
 #pragma unroll
-      for (int sb = 0; sb < 4; ++sb)
+      for (int j = 0; j < 4; ++j) down[sb][j] = sU[(16 * sb + 4 * g + j) * CS + n];
+    asm volatile("" ::: "memory");
 #pragma unroll
-        for (int j = 0; j < 4; ++j) s = mfma4(kt[i][sb][j], sU[(16 * sb + 4 * g + j) * CS + n], s);
-      S[i] = s;
-    }
-    if (c + 1 < chunks) fetch_second(c + 1);
+    for (int i = 0; i < RT; ++i) S[i] = S[i] * A.eg[i];
+#pragma unroll
+    for (int sb = 0; sb < 4; ++sb)
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+#pragma unroll
+        for (int i = 0; i < RT; ++i) S[i] = mfma4(A.kt[i][sb][j], down[sb][j], S[i]);
+    fetch_second(A, c + 2);
+  };
+  Ahead even, odd;
+  fetch_first(even, 0);                   // in the order in which the steps will ask, so that the waits agree
+  asm volatile("" ::: "memory");
+  fetch_second(even, 0);
+  asm volatile("" ::: "memory");
+  fetch_first(odd, 1);
+  asm volatile("" ::: "memory");
+  fetch_second(odd, 1);
+  asm volatile("" ::: "memory");
+  for (int c = 0; c < chunks; c += 2) {
+    step(even, c);
+    if (c + 1 < chunks) step(odd, c + 1);
   }
 #pragma unroll
   for (int i = 0; i < RT; ++i)
@@ -624,7 +663,7 @@ static int scan_launch(const DeltaArgs& a, int rows, hipStream_t s) {
   while (R < 64 && CB * ((a.d + R - 1) / R) > 16) R *= 2;
   const int RG = (a.d + R - 1) / R, waves = CB * RG;
   if (waves > 16) MIE_FAIL("gated_delta: states of %d x %d do not fit a workgroup", a.d, a.dv);
-  const size_t lds = ((size_t)3 * TB * RG * R + (size_t)4 * RG * CB * 64 + (size_t)TB * CB * 64 + 4 * TB) * sizeof(float);
+  const size_t lds = ((size_t)3 * TB * RG * R + (size_t)4 * RG * CB * 64 + (size_t)2 * TB * CB * 64 + 4 * TB) * sizeof(float);
   if (lds > 64 * 1024) MIE_FAIL("gated_delta: %zu bytes of LDS", lds);
 #define SCAN(R_) hipLaunchKernelGGL((scan_kernel<R_, TO>), dim3(rows, a.H), dim3(waves * 64), lds, s, a, CB)
   if (R == 8) SCAN(8);
@@ -638,7 +677,7 @@ static int scan_launch(const DeltaArgs& a, int rows, hipStream_t s) {
 
 template <int DP, typename TO>
 static int chunks_launch(const ChunkArgs& p, int rows, hipStream_t s) {
-  const size_t lds = ((size_t)3 * CH * (DP + 4) + (size_t)2 * CH * MS + CH) * sizeof(float);
+  const size_t lds = ((size_t)3 * CH * (DP + 4) + (size_t)2 * CH * MS + CH + 4 * DP) * sizeof(float);
   static bool allowed[64] = {};
   int dev = 0;
   if (hipGetDevice(&dev) != hipSuccess || dev < 0 || dev >= 64) MIE_FAIL("gated_delta: no current device");
@@ -647,8 +686,8 @@ static int chunks_launch(const ChunkArgs& p, int rows, hipStream_t s) {
     if (e != hipSuccess) MIE_FAIL("gated_delta: %zu bytes of LDS refused: %s", lds, hipGetErrorString(e));
     allowed[dev] = true;
   }
-  const dim3 units(rows * p.max_chunks, p.s.H);
-  hipLaunchKernelGGL(chunk_solve_kernel<DP>, units, dim3(256), lds, s, p);
+  const dim3 units(p.s.H, p.units < 32768 ? p.units : 32768, (p.units + 32767) / 32768);
+  hipLaunchKernelGGL(chunk_solve_kernel<DP>, units, dim3(SOLVE_THREADS), lds, s, p);
   MIE_CHECK_LAUNCH("gated_delta (chunks: solve)");
   hipLaunchKernelGGL(chunk_fold_kernel<DP>, dim3(p.s.H, rows, p.VP / 16), dim3(256), 0, s, p);
   MIE_CHECK_LAUNCH("gated_delta (chunks: fold)");
@@ -709,8 +748,8 @@ MIE_EXPORT int mie_gated_delta(const float* u, long ld_u, int q_col, int k_col, 
   if (max_chunks < 1 || !scratch || DP < d || VP < dv || (uintptr_t)scratch % 16) MIE_FAIL("gated_delta: chunks, %d a row, padded to %d x %d", max_chunks, DP, VP);
   if ((long)n * max_chunks > 2147483647L) MIE_FAIL("gated_delta: %d rows of %d chunks are beyond the grid", n, max_chunks);
   a.first_row = whole_rows;
-  const size_t units = (size_t)n * max_chunks * H;
-  ChunkArgs p{a, max_chunks, VP, nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, nullptr};
+  const size_t units = (size_t)n * max_chunks * H;      // of scratch
+  ChunkArgs p{a, max_chunks, n * max_chunks, VP, nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, nullptr};
   float* at = scratch;
   auto take = [&](size_t per) { float* q = at; at += units * per; return q; };
   p.W = take((size_t)CH * DP);

@@ -70,7 +70,7 @@ register_kernel_module("delta_rule", {
 register_kernel_module("gated_delta", {
     "mie_gated_delta": [P, L, I, I, I, P, L, I, I, I, P, I, P, P, P, I, F, P, F, P, P, P, P, P, P, I, I, I, I, I, I, I, I, I, I, I, P, P],
     "mie_gated_delta_unit_floats": [I, I],
-})
+}, flags=["-mllvm", "-amdgpu-mfma-vgpr-form"])
 register_kernel_module("gla", {
     "mie_gla": [P, L, I, I, I, I, I, P, I, P, F, F, P, F, P, P, P, P, P, I, I, I, I, I, I, I, I, P, P, P, P],
 })
