@@ -25,7 +25,14 @@
 typedef float f32x4 __attribute__((ext_vector_type(4)));
 constexpr float LOG2E = 1.4426950408889634f;
 
-__device__ __forceinline__ float softplus(float z) { return z > 20.f ? z : log1pf(expf(z)); }
+// max(z, 0) + log(1 + e), e = 2^(-|z| log2 e): with u = 1 + e as rounded, log(1 + e) = log(u) e / (u - 1) (Kahan's correction: what u
+// lost of e is made up by the factor), so the hardware's logarithm and reciprocal are enough
+__device__ __forceinline__ float softplus(float z) {
+  const float e = __builtin_amdgcn_exp2f(-fabsf(z) * LOG2E), u = 1.0f + e, d = u - 1.0f;
+  const float l = d == 0.f ? e : __builtin_amdgcn_logf(u) * 0.6931471805599453f * (e * __builtin_amdgcn_rcpf(d));
+  return fmaxf(z, 0.f) + l;
+}
+__device__ __forceinline__ float gate_sigmoid(float z) { return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-z * LOG2E)); }
 __device__ __forceinline__ float pow2(float x) { return __builtin_amdgcn_exp2f(x); }      // below 2^-126: 0
 // The waves meet over the LDS only: loads and stores of global memory stay on their way (__syncthreads would wait for them)
 __device__ __forceinline__ void lds_barrier() {
@@ -76,7 +83,7 @@ low_rank_kernel(const float* __restrict__ sums, long ld, int a_col, int g_col, c
     for (int e = 0; e < 4; ++e) {
       const int t = t0 + 16 * i + 4 * g + e;
       if (t >= tokens) continue;
-      if (is_gate) gate[(size_t)t * channels + c] = mie_sigmoid(acc[i][e]);
+      if (is_gate) gate[(size_t)t * channels + c] = gate_sigmoid(acc[i][e]);
       else la[(size_t)t * channels + c] = r * softplus(acc[i][e] + b);
     }
 }
