@@ -56,7 +56,7 @@ def _shape(vocab, width, heads, kv_heads, dim, chunk, delta_heads, delta_kv_head
            repeats, times):
     """A named size: ``repeats`` times the run (delta rule, attention, attention), the second layer of the first run looped
     ``times`` times with the third."""
-    rot = dict(base=50000.0, dims=dim // 2, scaling=dict(factor=4.0, original=4096, fast=32.0, slow=1.0))
+    rot = dict(base=10000.0, dims=dim // 2, scaling=dict(factor=4.0, original=4096, fast=32.0, slow=1.0))
     att = dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=dim, scale=dim ** -0.5, conv=4, mask=dict(size=chunk), rot=rot)
     delta = dict(heads=delta_heads, kv_heads=delta_kv_heads, dim=delta_dim, vdim=delta_vdim, conv=4, decay_rank=rank, gate_rank=rank)
     moe = dict(kind="moe", expert=dict(ff=expert_ff), router=dict(experts=experts, top=top, scale=2.0))
